@@ -423,31 +423,63 @@ OME_API int ome_diff_head_norm(const void* a, void* out, int T, int H, int R, in
 
 // Output gate of an attention layer: out[t, h * vdim + d] = o[t, h, d] * gate(g[t, h * vdim + d]),
 // d < vdim <= D (o's head rows are D wide; the padding beyond vdim is dropped).  kind 0: sigmoid,
-// 1: SiLU.
+// 1: SiLU.  per_head: g has one number per head instead (row stride g_stride).
 template <typename T>
 __global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ o, const T* __restrict__ g,
                                                         int64_t g_stride, T* __restrict__ out, int H, int D,
-                                                        int vdim, int kind) {
+                                                        int vdim, int kind, int per_head) {
   const int64_t t = blockIdx.x;
   const int n = H * vdim;
   for (int i = threadIdx.x; i < n; i += 256) {
     const int h = i / vdim, d = i - h * vdim;
-    const float gv = (float)g[t * g_stride + i];
+    const float gv = (float)g[t * g_stride + (per_head ? h : i)];
     const float sg = 1.f / (1.f + expf(-gv));
     out[t * n + i] = (T)((float)o[(t * H + h) * D + d] * (kind == 0 ? sg : gv * sg));
   }
 }
 
+// bf16 rows of 8-element vectors: one per thread (vdim % 8 == 0, D % 8 == 0, 16-byte aligned rows)
+__global__ __launch_bounds__(256) void head_gate_vec_kernel(const bf16* __restrict__ o, const bf16* __restrict__ g,
+                                                            int64_t g_stride, bf16* __restrict__ out, int H, int D,
+                                                            int vdim, int kind, int per_head, int64_t total) {
+  const int64_t v = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (v >= total) return;
+  const int nv = H * vdim / 8;
+  const int64_t t = v / nv;
+  const int i = (int)(v - t * nv) * 8;
+  const int h = i / vdim, d = i - h * vdim;
+  const bf16x8 x = ld8(o + (t * H + h) * D + d);
+  bf16x8 gv = {};
+  float g1 = 0.f;
+  if (per_head) g1 = (float)g[t * g_stride + h];
+  else gv = ld8(g + t * g_stride + i);
+  bf16x8 r;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float z = per_head ? g1 : (float)gv[e];
+    const float sg = 1.f / (1.f + expf(-z));
+    r[e] = (bf16)((float)x[e] * (kind == 0 ? sg : z * sg));
+  }
+  st8(out + t * H * vdim + i, r);
+}
+
 OME_API int ome_head_gate(const void* o, const void* g, int64_t g_stride, void* out, int T, int H, int D, int vdim,
-                          int kind, int f32, hipStream_t stream) {
+                          int kind, int f32, int per_head, hipStream_t stream) {
   if (T <= 0) return 0;
   if (vdim <= 0 || vdim > D) return -2;
-  if (f32)
+  const bool al = (((uintptr_t)o | (uintptr_t)out) & 15) == 0 &&
+                  (per_head || (((uintptr_t)g & 15) == 0 && g_stride % 8 == 0));
+  if (!f32 && vdim % 8 == 0 && D % 8 == 0 && al) {
+    const int64_t total = (int64_t)T * (H * vdim / 8);
+    head_gate_vec_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(
+        (const bf16*)o, (const bf16*)g, g_stride, (bf16*)out, H, D, vdim, kind, per_head, total);
+  } else if (f32) {
     head_gate_kernel<float><<<T, 256, 0, stream>>>((const float*)o, (const float*)g, g_stride, (float*)out, H, D, vdim,
-                                                   kind);
-  else
+                                                   kind, per_head);
+  } else {
     head_gate_kernel<bf16><<<T, 256, 0, stream>>>((const bf16*)o, (const bf16*)g, g_stride, (bf16*)out, H, D, vdim,
-                                                  kind);
+                                                  kind, per_head);
+  }
   OME_CHECK_LAUNCH();
   return 0;
 }

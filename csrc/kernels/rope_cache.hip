@@ -485,7 +485,11 @@ OME_API int ome_wide_norm_rope_cache(const void* q, int64_t q_stride, const void
 // (unit_norm; no weight).  q goes to q_out [T, Hq, D], k / v into the paged cache (K [pages, Hkv,
 // P, D], V [pages, Hkv, D, P]); head tails beyond dim / vdim are written as zeros (q, k) or left
 // as the cache's zeros (v).  Convolution sum, angles, rotation and norm are fp32; one rounding at
-// the store.
+// the store.  Optional: biases of the three projections (added before the convolution; `tail` keeps
+// the projections WITHOUT them, rows before the sequence's position 0 stay zero), a weighted RMS
+// norm per head BEFORE the rotation (weights of width dim shared by the heads), a value mix v <-
+// (1 - lam) v + lam v_first (lam: one fp32 number in memory) and a copy of the values to v_out
+// (v_first / v_out: dense [T, Hkv * vdim]).
 //
 // The last K-1 projected rows of every sequence live in `tail` [slots, K-1, C] (C = all q, k, v
 // channels; row j = input at time -(K-1) + j of the next step).  Time is tiled: one workgroup =
@@ -498,6 +502,16 @@ namespace {
 constexpr int CR_TILE = 32;
 constexpr int CR_MAXS = 1024;   // sequence starts staged in LDS (more: read from global memory)
 
+// optional parts of the step (null = absent)
+template <typename T>
+struct ConvRopeExtra {
+  const T *bq, *bk, *bv;     // projection biases
+  const T *qn, *kn;          // per-head norm weights [dim], before the rotation
+  const float* lam;          // value mix: one number
+  const T* v_first;          // [T, Hkv * vdim]
+  T* v_out;                  // [T, Hkv * vdim]
+};
+
 template <typename T>
 __global__ __launch_bounds__(256) void conv_rope_cache_kernel(
     const T* __restrict__ q, int64_t q_stride, const T* __restrict__ k, int64_t k_stride, const T* __restrict__ v,
@@ -505,7 +519,7 @@ __global__ __launch_bounds__(256) void conv_rope_cache_kernel(
     T* __restrict__ tail, const int* __restrict__ cu, const int* __restrict__ slot, const int* __restrict__ reset,
     const int* __restrict__ positions, const float* __restrict__ cos_sin, int rot_dim, int interleaved,
     int unit_norm, float eps, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
-    const int* __restrict__ slots, int Hq, int Hkv, int dim, int vdim, int D, int P, int S) {
+    const int* __restrict__ slots, int Hq, int Hkv, int dim, int vdim, int D, int P, int S, ConvRopeExtra<T> ex) {
   extern __shared__ float sm[];   // [CR_TILE + K - 1][d] input rows, then [K][d] taps
   const int hh = blockIdx.x;
   // blockIdx.y counts the tiles of all sequences in turn (the grid is the upper bound T / CR_TILE + S);
@@ -618,6 +632,16 @@ __global__ __launch_bounds__(256) void conv_rope_cache_kernel(
       tl[(int64_t)j * C + c] = t >= 0 ? src[(int64_t)(r0 + t) * sstride + head * d + c] : (T)rows[(KT + t) * d + c];
     }
   }
+  const T* bias = kind == 0 ? ex.bq : (kind == 1 ? ex.bk : ex.bv);
+  const T* nw = kind == 0 ? ex.qn : ex.kn;
+  float bc[4], nc[4];   // this lane's biases and norm weights
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int c = (u >> 1) * 128 + 2 * lane + (u & 1);
+    bc[u] = bias != nullptr && c < d ? (float)bias[head * d + c] : 0.f;
+    nc[u] = kind != 2 && nw != nullptr && c < d ? (float)nw[c] : 1.f;
+  }
+  const float lam = kind == 2 && ex.lam != nullptr ? ex.lam[0] : 0.f;
   // a lane owns two pairs of neighbouring channels: register u <-> channel (u >> 1) * 128 + 2 lane + (u & 1)
   // (d <= 256), so an interleaved rotary pair sits in one lane and stores are 4 bytes wide
 #pragma unroll
@@ -633,14 +657,21 @@ __global__ __launch_bounds__(256) void conv_rope_cache_kernel(
       const int c = (u >> 1) * 128 + 2 * lane + (u & 1);
       float acc = 0.f;
       if (c < d) {
-        if (K > 0)
-          for (int j = 0; j < K; ++j) acc += taps[j * d + c] * rows[(rr + j) * d + c];
+        if (K > 0)   // (the bias belongs to the rows of the sequence only, not to the zeros before it)
+          for (int j = 0; j < K; ++j) acc += taps[j * d + c] * (rows[(rr + j) * d + c] + (pos - KT + j >= 0 ? bc[u] : 0.f));
         else
-          acc = rows[rr * d + c];
+          acc = rows[rr * d + c] + bc[u];
       }
       y[u] = acc;
     }
     if (kind == 2) {
+      const int64_t vrow = ((int64_t)r * Hkv + head) * vdim;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int c = (u >> 1) * 128 + 2 * lane + (u & 1);
+        if (c < d && ex.lam != nullptr) y[u] = (1.f - lam) * y[u] + lam * (float)ex.v_first[vrow + c];
+        if (c < d && ex.v_out != nullptr) ex.v_out[vrow + c] = (T)y[u];
+      }
       if (slot_t >= 0) {
         T* vc = v_cache + (((int64_t)(slot_t / P) * Hkv + head) * D) * P + slot_t % P;
 #pragma unroll
@@ -650,6 +681,14 @@ __global__ __launch_bounds__(256) void conv_rope_cache_kernel(
         }
       }
       continue;
+    }
+    if (nw != nullptr) {
+      float ss = 0.f;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) ss += y[u] * y[u];   // (channels beyond d hold zeros)
+      const float rs = 1.f / sqrtf(wave_sum(ss) / (float)d + eps);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) y[u] *= rs * nc[u];
     }
     if (rot_dim > 0) {
       if (interleaved) {
@@ -719,7 +758,7 @@ __global__ __launch_bounds__(256) void conv_rope_cache_kernel(
 
 // ------------------------------------------------------------------------------------------
 // The same step for the common shapes (head widths in multiples of 8, up to CV_MAXK taps,
-// interleaved rotary pairs, 16-byte aligned rows), without LDS and without barriers: one item =
+// interleaved rotary pairs, or halves of a multiple of 8 channels; 16-byte aligned rows), without LDS and without barriers: one item =
 // (row, head of q / k / v), a lane owns 8 neighbouring channels (D / 8 lanes per item), reads its K
 // input vectors straight from the projection rows (L1 / L2 keep the K-fold reuse) or, for rows
 // before the step's first, from the sequence's tail, and writes 16-byte vectors.  Per row the
@@ -762,9 +801,9 @@ __global__ __launch_bounds__(256) void conv_rope_cache_vec_kernel(
     const T* __restrict__ q, int64_t q_stride, const T* __restrict__ k, int64_t k_stride, const T* __restrict__ v,
     int64_t v_stride, const T* __restrict__ wq, const T* __restrict__ wk, const T* __restrict__ wv,
     const T* __restrict__ tail, const int* __restrict__ row_start, const int* __restrict__ row_slot,
-    const int* __restrict__ positions, const float* __restrict__ cos_sin, int rot_dim, int unit_norm, float eps,
-    T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, const int* __restrict__ slots, int Tn,
-    int Hq, int Hkv, int dim, int vdim, int P) {
+    const int* __restrict__ positions, const float* __restrict__ cos_sin, int rot_dim, int interleaved, int unit_norm,
+    float eps, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, const int* __restrict__ slots,
+    int Tn, int Hq, int Hkv, int dim, int vdim, int P, ConvRopeExtra<T> ex) {
   constexpr int D = GS * 8, KT = K > 0 ? K - 1 : 0, KK = K > 0 ? K : 1;
   const int Ht = Hq + 2 * Hkv;
   const int64_t item = (int64_t)blockIdx.x * (256 / GS) + threadIdx.x / GS;
@@ -801,6 +840,15 @@ __global__ __launch_bounds__(256) void conv_rope_cache_vec_kernel(
     }
   }
   float y[8];
+  const T* bias = kind == 0 ? ex.bq : (kind == 1 ? ex.bk : ex.bv);
+  if (bias != nullptr && on) {   // (rows before the sequence's position 0 are zeros, without the bias)
+    float b[8];
+    cv_ld8<T>(bias + head * d + c8, b);
+#pragma unroll
+    for (int j = 0; j < KK; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[j][e] += pos - KT + j >= 0 ? b[e] : 0.f;
+  }
   if constexpr (K > 0) {
     if (on) {   // this lane's taps are contiguous: w[e * K + j]
 #pragma unroll
@@ -823,6 +871,15 @@ __global__ __launch_bounds__(256) void conv_rope_cache_vec_kernel(
     for (int e = 0; e < 8; ++e) y[e] = x[0][e];
   }
   if (kind == 2) {
+    const int64_t vo = ((int64_t)t * Hkv + head) * vdim + c8;
+    if (on && ex.lam != nullptr) {
+      const float lam = ex.lam[0];
+      float f[8];
+      cv_ld8<T>(ex.v_first + vo, f);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y[e] = (1.f - lam) * y[e] + lam * f[e];
+    }
+    if (on && ex.v_out != nullptr) cv_st8<T>(ex.v_out + vo, y);
     if (on && slot_t >= 0) {
       T* vc = v_cache + (((int64_t)(slot_t / P) * Hkv + head) * D + c8) * P + slot_t % P;
 #pragma unroll
@@ -830,7 +887,36 @@ __global__ __launch_bounds__(256) void conv_rope_cache_vec_kernel(
     }
   }
   // (q / k from here; lanes of value items only take part in the shuffles)
-  if (kind != 2 && on && rot_dim > 0) {
+  if (ex.qn != nullptr) {   // weighted norm per head before the rotation
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += y[e] * y[e];
+#pragma unroll
+    for (int o = GS / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+    const float rsq = 1.f / sqrtf(ss / (float)d + eps);
+    if (kind != 2 && on) {
+      float nw[8];
+      cv_ld8<T>((kind == 0 ? ex.qn : ex.kn) + c8, nw);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y[e] *= rsq * nw[e];
+    }
+  }
+  if (rot_dim > 0 && !interleaved) {   // pairs (i, i + half): the partner's channels sit half / 8 lanes away
+    const int half = rot_dim >> 1, h8 = half >> 3;
+    const bool lo = l < h8, in = l < 2 * h8;
+    const int pl = (int)(threadIdx.x & 63) + (in ? (lo ? h8 : -h8) : 0);
+    float other[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) other[e] = __shfl(y[e], pl);
+    if (kind != 2 && on && in) {
+      const float* cs = cos_sin + (int64_t)pos * rot_dim + (lo ? c8 : c8 - half);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float co = cs[e], si = cs[half + e];
+        y[e] = lo ? y[e] * co - other[e] * si : y[e] * co + other[e] * si;
+      }
+    }
+  } else if (kind != 2 && on && rot_dim > 0) {
     const float* cs = cos_sin + (int64_t)pos * rot_dim;
     const int half = rot_dim >> 1;
 #pragma unroll
@@ -895,25 +981,32 @@ OME_API int ome_conv_rope_cache_vec(const void* q, int64_t q_stride, const void*
                                     int64_t v_stride, const void* wq, const void* wk, const void* wv, int K,
                                     void* tail, const int* cu, const int* slot, const int* reset, int S,
                                     const int* row_start, const int* row_slot, const int* positions,
-                                    const float* cos_sin, int rot_dim, int unit_norm, float eps, void* q_out,
-                                    void* k_cache, void* v_cache, const int* slots, int T, int Hq, int Hkv, int dim,
-                                    int vdim, int D, int P, int f32, hipStream_t stream) {
+                                    const float* cos_sin, int rot_dim, int interleaved, int unit_norm, float eps,
+                                    void* q_out, void* k_cache, void* v_cache, const int* slots, int T, int Hq, int Hkv,
+                                    int dim, int vdim, int D, int P, const void* bq, const void* bk, const void* bv,
+                                    const void* qn, const void* kn, const float* lam, const void* v_first, void* v_out,
+                                    int f32, hipStream_t stream) {
   if (T <= 0 || S <= 0) return 0;
   const int esz = f32 ? 4 : 2;
   auto al = [&](const void* p, int64_t stride) { return (((uintptr_t)p | (uintptr_t)(stride * esz)) & 15) == 0; };
   if (K < 0 || K > CV_MAXK || dim % 8 || vdim % 8 || dim > D || vdim > D || (D != 64 && D != 128 && D != 256) ||
       (rot_dim & 1) || rot_dim > dim || !al(q, q_stride) || !al(k, k_stride) || !al(v, v_stride) || !al(wq, 0) ||
-      !al(wk, 0) || !al(wv, 0) || !al(tail, 0) || !al(q_out, 0) || !al(k_cache, 0) ||
+      !al(wk, 0) || !al(wv, 0) || !al(tail, 0) || !al(q_out, 0) || !al(k_cache, 0) || !al(bq, 0) || !al(bk, 0) ||
+      !al(bv, 0) || !al(qn, 0) || !al(kn, 0) || !al(v_first, 0) || !al(v_out, 0) ||
+      (rot_dim > 0 && !interleaved && rot_dim % 16) ||
       (((int64_t)(Hq + Hkv) * dim + (int64_t)Hkv * vdim) * esz) % 16)
     return -9;
-  if (K > 1 && tail == nullptr) return -2;
+  if ((K > 1 && tail == nullptr) || (lam != nullptr && v_first == nullptr) || ((qn == nullptr) != (kn == nullptr)))
+    return -2;
   const int gs = D / 8;
   const int64_t items = (int64_t)T * (Hq + 2 * Hkv);
   const unsigned grid = (unsigned)((items + 256 / gs - 1) / (256 / gs));
 #define CV_ARGS(TT)                                                                                                 \
   (const TT*)q, q_stride, (const TT*)k, k_stride, (const TT*)v, v_stride, (const TT*)wq, (const TT*)wk,            \
-      (const TT*)wv, (const TT*)tail, row_start, row_slot, positions, cos_sin, rot_dim, unit_norm, eps, (TT*)q_out, \
-      (TT*)k_cache, (TT*)v_cache, slots, T, Hq, Hkv, dim, vdim, P
+      (const TT*)wv, (const TT*)tail, row_start, row_slot, positions, cos_sin, rot_dim, interleaved, unit_norm,    \
+      eps, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, slots, T, Hq, Hkv, dim, vdim, P,                                 \
+      ConvRopeExtra<TT>{(const TT*)bq, (const TT*)bk, (const TT*)bv, (const TT*)qn, (const TT*)kn, lam,            \
+                        (const TT*)v_first, (TT*)v_out}
 #define CV_GS(TT, KK)                                                                                   \
   do {                                                                                                  \
     if (gs == 8) conv_rope_cache_vec_kernel<TT, KK, 8><<<grid, 256, 0, stream>>>(CV_ARGS(TT));          \
@@ -957,11 +1050,14 @@ OME_API int ome_conv_rope_cache(const void* q, int64_t q_stride, const void* k, 
                                 const int* cu, const int* slot, const int* reset, int S, const int* positions,
                                 const float* cos_sin, int rot_dim, int interleaved, int unit_norm, float eps,
                                 void* q_out, void* k_cache, void* v_cache, const int* slots, int T, int Hq, int Hkv,
-                                int dim, int vdim, int D, int P, int f32, hipStream_t stream) {
+                                int dim, int vdim, int D, int P, const void* bq, const void* bk, const void* bv,
+                                const void* qn, const void* kn, const float* lam, const void* v_first, void* v_out,
+                                int f32, hipStream_t stream) {
   if (T <= 0 || S <= 0) return 0;
   if (dim <= 0 || vdim <= 0 || dim > D || vdim > D || D > 256 || K < 0 || K > 33 || rot_dim > dim || (rot_dim & 1))
     return -2;
   if (K > 0 && (wq == nullptr || wk == nullptr || wv == nullptr || (K > 1 && tail == nullptr))) return -2;
+  if ((lam != nullptr && v_first == nullptr) || ((qn == nullptr) != (kn == nullptr))) return -2;
   const int tiles = (T + CR_TILE - 1) / CR_TILE + S;
   if (tiles > 65535) return -3;
   const int dmax = dim > vdim ? dim : vdim;
@@ -980,7 +1076,9 @@ OME_API int ome_conv_rope_cache(const void* q, int64_t q_stride, const void* k, 
     conv_rope_cache_kernel<TT><<<grid, 256, lds, stream>>>(                                                         \
         (const TT*)q, q_stride, (const TT*)k, k_stride, (const TT*)v, v_stride, (const TT*)wq, (const TT*)wk,       \
         (const TT*)wv, K, (TT*)tail, cu, slot, reset, positions, cos_sin, rot_dim, interleaved, unit_norm, eps,     \
-        (TT*)q_out, (TT*)k_cache, (TT*)v_cache, slots, Hq, Hkv, dim, vdim, D, P, S);                                \
+        (TT*)q_out, (TT*)k_cache, (TT*)v_cache, slots, Hq, Hkv, dim, vdim, D, P, S,                                \
+        ConvRopeExtra<TT>{(const TT*)bq, (const TT*)bk, (const TT*)bv, (const TT*)qn, (const TT*)kn, lam,          \
+                          (const TT*)v_first, (TT*)v_out});                                                        \
   } while (0)
   if (f32) CRC_LAUNCH(float);
   else CRC_LAUNCH(bf16);

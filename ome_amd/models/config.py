@@ -169,7 +169,7 @@ def layer_runs(c: dict[str, Any]) -> list[tuple[int, int]]:
 
 
 def _layer_list_keys(c: dict[str, Any]) -> dict[str, Any]:
-    """Layer-list configs (``architecture: Zavilorn`` / ``Metitar`` / ``Milenex`` / ``Nivasun``): ``layers`` is a
+    """Layer-list configs (``architecture: Zavilorn`` / ``Metitar`` / ``Milenex`` / ``Nivasun`` / ``Pagatar``): ``layers`` is a
     list of blocks, each with its mixer ``type``, the mixer's own sizes and its feed-forward.  The
     standard keys describe the envelope the runtime sizes its workspaces by (widest attention layer,
     fewest kv heads); the model reads the per-layer entries from ``extra``.  ``num_hidden_layers``

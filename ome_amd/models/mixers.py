@@ -18,6 +18,11 @@ constructor argument), for decoders that assemble their layers from a per-layer 
   expert's input, plus an optional always-on shared expert;
 * :class:`TokenSideInput` -- a gated per-layer slice of a second token embedding, projected back to
   the stream;
+* :class:`ConvRotaryAttention` -- grouped-query attention behind short causal convolutions, with a
+  sliding window or chunks, optional biases, q / k norms before or after the rotation, sinks, value
+  mixing with an earlier layer and an output gate;
+* :class:`MinGruMixer` -- minGRU: an element-wise gated recurrence (fp32 state per request slot);
+* :class:`GroupRoutedMoE` -- softmax- or sigmoid-routed mixture of gated experts;
 * :class:`KeyValuedAttention` -- grouped-query attention whose values are the unrotated keys, with
   a per-head temperature, a sliding window and a softmax sink;
 * :class:`DifferentialAttention` -- two softmax maps per head over the same values, the second
@@ -298,18 +303,23 @@ class LatentAttention(_Block):
     its own W_uk / W_uv.  ``rot_dim`` = 0: no rotated part at all (no positions).  ``window`` > 0:
     query i sees keys j with 0 <= i - j < window.  ``sink`` False: an ordinary softmax.  ``gated``:
     the concatenated heads are multiplied by sigmoid(W_g h) before W_o (W_g rides in the fused
-    input projection).  Checkpoint tensors ``dq dq.norm uq [dkv dkv.norm] uk uv [sink] [g] o``."""
+    input projection); ``gated="head"``: W_g has one row per head, whose sigmoid multiplies the
+    head's whole output.  ``interleaved``: rotary pairs are (2i, 2i+1) -- the rows of W_uq and W_dkv
+    that make the rotated parts are reordered at load into the half-split order the kernels use
+    (queries and keys alike, so every dot product keeps its value).  Checkpoint tensors ``dq dq.norm uq [dkv dkv.norm] uk uv [sink] [g] o``."""
 
     HEAD_GROUP = 16   # query heads per kv head one launch of the generic attention kernels takes
 
     def __init__(self, layer: int, kv_layer: int, width: int, heads: int, dim: int, rot_dim: int, vdim: int,
                  kv_rank: int, q_rank: int, rot_base: float, rot_scaling: dict | None, scale: float, eps: float,
                  max_positions: int, device, dtype, latent_cache: bool | None = None, window: int = -1,
-                 sink: bool = True, gated: bool = False):
+                 sink: bool = True, gated: bool | str = False, interleaved: bool = False):
         super().__init__(device, dtype)
         if rot_dim % 2 or rot_dim < 0:
             raise ValueError(f"latent attention: rotary width {rot_dim} must be even")
         self.window, self.has_sink, self.gated = int(window) if window and window > 0 else -1, bool(sink), bool(gated)
+        self.ng = 0 if not gated else (heads if gated == "head" else heads * vdim)     # rows of W_g
+        self.interleaved = bool(interleaved)
         self.layer, self.kv_layer, self.width, self.H = layer, kv_layer, width, heads
         self.dim, self.rot, self.vdim, self.R, self.qr = dim, rot_dim, vdim, kv_rank, q_rank
         self.scale, self.eps = float(scale), float(eps)
@@ -332,9 +342,18 @@ class LatentAttention(_Block):
 
     def load(self, t: dict) -> None:
         H, R = self.H, self.R
-        parts = [t["dq"]] + ([t["dkv"]] if self.own_cache else []) + ([t["g"]] if self.gated else [])
+        uq, dkv = t["uq"], t["dkv"] if self.own_cache else None
+        if self.interleaved and self.rot:
+            order = torch.cat([torch.arange(0, self.rot, 2), torch.arange(1, self.rot, 2)])
+            q3 = uq.view(H, self.dim + self.rot, -1)
+            uq = torch.cat([q3[:, :self.dim], q3[:, self.dim:][:, order]], 1).reshape(uq.shape)
+            if dkv is not None:
+                dkv = torch.cat([dkv[:R], dkv[R:][order]], 0)
+        if self.gated and t["g"].shape[0] != self.ng:
+            raise ValueError(f"latent attention: g has {t['g'].shape[0]} rows, {self.ng} expected")
+        parts = [t["dq"]] + ([dkv] if self.own_cache else []) + ([t["g"]] if self.gated else [])
         self.w_in = self._put(torch.cat(parts, 0))
-        self.qn, self.w_uq = self._put(t["dq.norm"]), self._put(t["uq"])
+        self.qn, self.w_uq = self._put(t["dq.norm"]), self._put(uq)
         if self.own_cache:
             self.kvn = self._put(t["dkv.norm"])
         self.w_uk = self._put(t["uk"].view(H, self.dim, R))                       # q_lat = q_nope @ W_uk[h]
@@ -344,8 +363,7 @@ class LatentAttention(_Block):
 
     def init_random(self, gen, std: float) -> None:
         H, R = self.H, self.R
-        self.w_in = self._rand(gen, self.qr + (R + self.rot if self.own_cache else 0) +
-                               (H * self.vdim if self.gated else 0), self.width, std=std)
+        self.w_in = self._rand(gen, self.qr + (R + self.rot if self.own_cache else 0) + self.ng, self.width, std=std)
         self.qn = torch.ones(self.qr, dtype=self.dtype, device=self.device)
         self.w_uq = self._rand(gen, H * (self.dim + self.rot), self.qr, std=std)
         if self.own_cache:
@@ -383,7 +401,7 @@ class LatentAttention(_Block):
         o = torch.empty(T, H * self.vdim, dtype=h.dtype, device=h.device)
         torch.bmm(o_lat[:, :, :R].transpose(0, 1), self.w_uv, out=o.view(T, H, self.vdim).transpose(0, 1))
         if self.gated:
-            o = ops.head_gate(o.view(T, H, self.vdim), a[:, a.shape[1] - H * self.vdim:], self.vdim, 0)
+            o = ops.head_gate(o.view(T, H, self.vdim), a[:, a.shape[1] - self.ng:], self.vdim, 0)
         return linear(o, self.w_o)
 
 
@@ -485,6 +503,19 @@ class PolyNormMLP(_Block):
         return linear(ops.polynorm(linear(h, self.w_up), self.coef, self.eps), self.w_d)
 
 
+def grouped_experts_ok(b) -> bool:
+    """Does this expert block run on the grouped MFMA GEMMs (bf16 on a GPU, widths in multiples of 32)?"""
+    return b.device.type == "cuda" and b.dtype == torch.bfloat16 and b.width % 32 == 0 and b.ff % 32 == 0
+
+
+def expert_layout(b) -> None:
+    """After ``w13`` [E, 2 ff, width] / ``w2`` [E, width, ff] are set: blocks on the dense path keep
+    the experts as contiguous [E, in, out] operands of the batched products instead (a transposed
+    view is never handed to a batched 16-bit GEMM)."""
+    if not grouped_experts_ok(b):
+        b.w13, b.w2 = b.w13.transpose(1, 2).contiguous(), b.w2.transpose(1, 2).contiguous()
+
+
 class InputScaledMoE(_Block):
     """Mixture of SwiGLU experts (no biases): router scores s = sigmoid(W_r h) from fp32 logits, the
     ``top`` largest chosen, weights = those scores (not renormalised) applied to the expert's INPUT:
@@ -505,6 +536,7 @@ class InputScaledMoE(_Block):
         self.w_router = self._put(t["router"])
         self.w13 = self._put(torch.stack([torch.cat([t[f"e{e}.gate"], t[f"e{e}.up"]], 0) for e in range(self.E)]))
         self.w2 = self._put(torch.stack([t[f"e{e}.down"] for e in range(self.E)]))
+        expert_layout(self)
         if self.sff:
             self.w_sgu, self.w_sd = self._put(torch.cat([t["shared.gate"], t["shared.up"]], 0)), self._put(t["shared.down"])
 
@@ -512,12 +544,13 @@ class InputScaledMoE(_Block):
         self.w_router = self._rand(gen, self.E, self.width, std=std)
         self.w13, self.w2 = self._rand(gen, self.E, 2 * self.ff, self.width, std=std), self._rand(
             gen, self.E, self.width, self.ff, std=std)
+        expert_layout(self)
         if self.sff:
             self.w_sgu, self.w_sd = self._rand(gen, 2 * self.sff, self.width, std=std), self._rand(
                 gen, self.width, self.sff, std=std)
 
     def grouped_ok(self, h: torch.Tensor) -> bool:
-        return h.is_cuda and h.dtype == torch.bfloat16 and self.width % 32 == 0 and self.ff % 32 == 0
+        return h.is_cuda and grouped_experts_ok(self)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         T, W = h.shape
@@ -531,9 +564,9 @@ class InputScaledMoE(_Block):
             return ops._combine(y, ones, inv, T, self.k, W, 1.0, sh.contiguous() if sh is not None else None)
         wd = torch.zeros(T, self.E, dtype=torch.float32, device=h.device).scatter_(1, tid.long(), tw)
         xe = (wd.t()[:, :, None] * h.float()[None]).to(h.dtype)           # [E, T, W]: s_e h, or 0
-        gu = torch.bmm(xe, self.w13.transpose(1, 2))
+        gu = torch.bmm(xe, self.w13)
         hh = ops.act_and_mul(gu.view(self.E * T, 2 * self.ff), 0).view(self.E, T, self.ff)
-        y = torch.bmm(hh, self.w2.transpose(1, 2)).float().sum(0)
+        y = torch.bmm(hh, self.w2).float().sum(0)
         return (y if sh is None else y + sh.float()).to(h.dtype)
 
 
@@ -566,46 +599,85 @@ def attention_rows(meta: AttnMeta, T: int) -> list:
     return [(s, e, bt, rows, lens - 1) for s, e, bt, rows, lens in latent_rows(meta, T)]
 
 
+def mask_window(size: int | None, chunked: bool) -> int:
+    """The attention kernels' ``window`` argument of a mask of ``size`` keys: a sliding window (> 0),
+    chunks counted from position 0 (< -1; chunks of one token = a window of one), or none (-1)."""
+    if not size or size <= 0:
+        return -1
+    return -int(size) if chunked and size > 1 else int(size)
+
+
 class ConvRotaryAttention(_Block):
     """Grouped-query attention whose q, k and v each pass a short causal depthwise convolution
     (``conv`` taps, no bias, no activation; 0: none) right after the projection; q and k are then
     rotated on the first ``rot_dims`` dims of every head (interleaved or half-split pairs) and,
-    after the rotation, divided by their root mean square per head (no weight); score = q.k *
-    ``scale``; query i sees keys j with 0 <= i - j < ``window``; softmax whose denominator also
-    holds exp(``sink``_h); W_o.  Checkpoint tensors ``q k v [q.conv k.conv v.conv] sink o``;
-    state: the last conv - 1 projected rows per request slot."""
+    after the rotation, divided by their root mean square per head (``unit_norm``; no weight); score
+    = q.k * ``scale``; query i sees keys j with 0 <= i - j < ``window``; softmax whose denominator
+    also holds exp(``sink``_h); W_o.  Checkpoint tensors ``q k v [q.conv k.conv v.conv] sink o``;
+    state: the last conv - 1 projected rows per request slot.
+
+    Options: ``bias`` -- q, k, v projections have biases (``q.b k.b v.b``), added before the
+    convolution.  ``head_norm`` -- RMS norm of every q / k head over ``dim`` with a weight shared by
+    the heads (``q.norm k.norm``), after the convolution and BEFORE the rotation.  ``rot_scaling``
+    -- YaRN (``config.yarn_rope_table``).  ``chunked`` -- the mask's size is a chunk: query i sees
+    keys j <= i with floor(i / size) = floor(j / size), chunks counted from position 0.  ``sink``
+    False -- an ordinary softmax.  ``gated`` -- the concatenated heads times sigmoid(W_g h) (``g``)
+    before W_o.  ``v_mix`` -- ``"first"``: this layer's values (after the convolution) are handed to
+    later layers of the same step; ``"mix"``: v <- (1 - lam) v + lam v_first with lam = ``vmix``,
+    and the mixed v is what is cached."""
 
     def __init__(self, layer: int, width: int, heads: int, kv_heads: int, dim: int, vdim: int, window: int,
                  conv: int, rot_base: float, rot_dims: int, scale: float, eps: float, max_positions: int, device,
-                 dtype, interleaved: bool = True, unit_norm: bool = True):
+                 dtype, interleaved: bool = True, unit_norm: bool = True, rot_scaling: dict | None = None,
+                 chunked: bool = False, bias: bool = False, head_norm: bool = False, sink: bool = True,
+                 gated: bool = False, v_mix: str | None = None):
         super().__init__(device, dtype)
-        if heads % kv_heads or heads // kv_heads > 16:
-            raise ValueError(f"attention: {heads} query heads over {kv_heads} kv heads (groups of <= 16 supported)")
+        if heads % kv_heads:
+            raise ValueError(f"attention: {heads} query heads do not divide over {kv_heads} kv heads")
         self.layer, self.width, self.Hq, self.Hkv, self.dim, self.vdim = layer, width, heads, kv_heads, dim, vdim
-        self.window, self.K = int(window) if window and window > 0 else -1, int(conv or 0)
+        self.window, self.K = mask_window(window, chunked), int(conv or 0)
         self.rot_dims, self.scale, self.eps = int(rot_dims), float(scale), float(eps)
         self.interleaved, self.unit_norm = interleaved, unit_norm
+        self.has_bias, self.head_norm, self.has_sink, self.gated, self.v_mix = bias, head_norm, sink, gated, v_mix
         self.D = attn_tile_dim(max(dim, vdim))
-        self.cos_sin = plain_rope_table(rot_base, self.rot_dims, max_positions, self.device) if rot_dims else \
+        self.cos_sin = yarn_rope_table(rot_base, self.rot_dims, max_positions, rot_scaling, self.device) if rot_dims else \
             torch.zeros(max_positions, 0, device=self.device)
         self.nq, self.nk, self.nv = heads * dim, kv_heads * dim, kv_heads * vdim
         self.w_in = self.cq = self.ck = self.cv = self.sink = self.w_o = None
+        self.bq = self.bk = self.bv = self.qn = self.kn = self.lam = None
         self.tail = None
 
     def load(self, t: dict) -> None:
-        self.w_in = self._put(torch.cat([t["q"], t["k"], t["v"]], 0))
+        self.w_in = self._put(torch.cat([t["q"], t["k"], t["v"]] + ([t["g"]] if self.gated else []), 0))
+        rows = self.nq + self.nk + self.nv + (self.Hq * self.vdim if self.gated else 0)
+        if tuple(self.w_in.shape) != (rows, self.width):
+            raise ValueError(f"attention: projections {tuple(self.w_in.shape)} != [{rows}, {self.width}]")
         if self.K:
             self.cq, self.ck, self.cv = self._put(t["q.conv"]), self._put(t["k.conv"]), self._put(t["v.conv"])
             for n, c, w in (("q", self.nq, self.cq), ("k", self.nk, self.ck), ("v", self.nv, self.cv)):
                 if tuple(w.shape) != (c, self.K):
                     raise ValueError(f"{n}.conv: shape {tuple(w.shape)} != [{c}, {self.K}]")
-        self.sink, self.w_o = self._put(t["sink"], torch.float32), self._put(t["o"])
+        if self.has_bias:
+            self.bq, self.bk, self.bv = self._put(t["q.b"]), self._put(t["k.b"]), self._put(t["v.b"])
+        if self.head_norm:
+            self.qn, self.kn = self._put(t["q.norm"]), self._put(t["k.norm"])
+        if self.v_mix == "mix":
+            self.lam = self._put(t["vmix"].reshape(1), torch.float32)
+        self.sink = self._put(t["sink"], torch.float32) if self.has_sink else None
+        self.w_o = self._put(t["o"])
 
     def init_random(self, gen, std: float) -> None:
-        self.w_in = self._rand(gen, self.nq + self.nk + self.nv, self.width, std=std)
+        self.w_in = self._rand(gen, self.nq + self.nk + self.nv + (self.Hq * self.vdim if self.gated else 0), self.width,
+                               std=std)
         if self.K:
             self.cq, self.ck, self.cv = (self._rand(gen, c, self.K, std=0.5) for c in (self.nq, self.nk, self.nv))
-        self.sink = torch.zeros(self.Hq, dtype=torch.float32, device=self.device)
+        if self.has_bias:
+            self.bq, self.bk, self.bv = (self._rand(gen, c, std=std) for c in (self.nq, self.nk, self.nv))
+        if self.head_norm:
+            self.qn, self.kn = (torch.ones(self.dim, dtype=self.dtype, device=self.device) for _ in range(2))
+        if self.v_mix == "mix":
+            self.lam = torch.full((1,), 0.3, dtype=torch.float32, device=self.device)
+        self.sink = torch.zeros(self.Hq, dtype=torch.float32, device=self.device) if self.has_sink else None
         self.w_o = self._rand(gen, self.width, self.Hq * self.vdim, std=std)
 
     def alloc_state(self, slots: int) -> None:
@@ -614,20 +686,63 @@ class ConvRotaryAttention(_Block):
 
     def forward(self, h: torch.Tensor, ctx: MixerCtx) -> torch.Tensor:
         T = h.shape[0]
-        nq, nk = self.nq, self.nk
-        p = linear(h, self.w_in)                                   # [T, q | k | v]
+        nq, nk, nv = self.nq, self.nk, self.nv
+        p = linear(h, self.w_in)                                   # [T, q | k | v (| gate)]
         q = torch.empty(T, self.Hq, self.D, dtype=h.dtype, device=h.device)
         k_cache, v_cache = ctx.kv.layer(self.layer)
         rows = ctx.cache.get("rows")
         if rows is None and h.is_cuda:
             rows = ctx.cache["rows"] = ops.seq_rows(ctx.seqs, T)
-        ops.conv_rope_cache(p[:, :nq], p[:, nq:nq + nk], p[:, nq + nk:], self.cq, self.ck, self.cv, self.tail, ctx.seqs,
-                            ctx.meta.positions, self.cos_sin, self.rot_dims, self.interleaved, self.unit_norm, self.eps,
-                            q, k_cache, v_cache, ctx.meta.slots, self.Hq, self.Hkv, self.dim, self.vdim, rows=rows)
+        v_out = None
+        if self.v_mix == "first":
+            v_out = ctx.cache["v_first"] = torch.empty(T, nv, dtype=h.dtype, device=h.device)
+        ops.conv_rope_cache(p[:, :nq], p[:, nq:nq + nk], p[:, nq + nk:nq + nk + nv], self.cq, self.ck, self.cv, self.tail,
+                            ctx.seqs, ctx.meta.positions, self.cos_sin, self.rot_dims, self.interleaved, self.unit_norm,
+                            self.eps, q, k_cache, v_cache, ctx.meta.slots, self.Hq, self.Hkv, self.dim, self.vdim, rows=rows,
+                            bias=(self.bq, self.bk, self.bv) if self.has_bias else None,
+                            head_norm=(self.qn, self.kn) if self.head_norm else None,
+                            v_mix=(self.lam, ctx.cache["v_first"]) if self.v_mix == "mix" else None, v_out=v_out)
         a = paged_attention(q, k_cache, v_cache, ctx.meta, self.scale, self.window, 0, self.sink)
+        if self.gated:
+            return linear(ops.head_gate(a, p[:, nq + nk + nv:], self.vdim, 0), self.w_o)
         if self.D != self.vdim:
             a = a[:, :, :self.vdim].reshape(T, self.Hq * self.vdim)
         return linear(a.view(T, self.Hq * self.vdim), self.w_o)
+
+
+class MinGruMixer(_Block):
+    """minGRU.  z = sigmoid(W_z h + b_z), u = W_x h + b_x, candidate c = u + 1/2 where u >= 0 and
+    sigmoid(u) where u < 0; S_t = (1 - z) S_{t-1} + z c element by element (``inner`` channels);
+    W_o (S_t * silu(W_g h)).  Checkpoint tensors ``z z.b x x.b g o``; state S [slots, inner] fp32.
+    Biases, activations, the recurrence and the gate are one op (``ops.mingru_scan``)."""
+
+    def __init__(self, width: int, inner: int, device, dtype):
+        super().__init__(device, dtype)
+        self.width, self.inner = width, inner
+        self.w_in = self.zb = self.xb = self.w_o = None
+        self.state = None
+
+    def load(self, t: dict) -> None:
+        self.w_in = self._put(torch.cat([t["z"], t["x"], t["g"]], 0))
+        if tuple(self.w_in.shape) != (3 * self.inner, self.width):
+            raise ValueError(f"mingru: z / x / g {tuple(self.w_in.shape)} != [3 * {self.inner}, {self.width}]")
+        self.zb, self.xb, self.w_o = self._put(t["z.b"]), self._put(t["x.b"]), self._put(t["o"])
+
+    def init_random(self, gen, std: float) -> None:
+        self.w_in = self._rand(gen, 3 * self.inner, self.width, std=std)
+        self.zb = torch.linspace(-4.0, 1.0, self.inner, device=self.device).to(self.dtype)
+        self.xb = torch.zeros(self.inner, dtype=self.dtype, device=self.device)
+        self.w_o = self._rand(gen, self.width, self.inner, std=std)
+
+    def alloc_state(self, slots: int) -> None:
+        self.state = torch.zeros(slots, self.inner, dtype=torch.float32, device=self.device)
+
+    def forward(self, h: torch.Tensor, ctx: MixerCtx) -> torch.Tensor:
+        n = self.inner
+        p = linear(h, self.w_in)                                          # [T, z | x | g]
+        o = ops.mingru_scan(p[:, :n], p[:, n:2 * n], p[:, 2 * n:], self.zb, self.xb, self.state, *ctx.seqs,
+                            single_rows=ctx.meta.is_decode)
+        return linear(o, self.w_o)
 
 
 class TalkingHeadsAttention(_Block):
@@ -723,6 +838,7 @@ class GroupRoutedMoE(_Block):
     chosen experts' outputs are weighted by their plain scores s (not renormalised).  An optional
     shared expert (own width and ``limit``) runs for every token, times sigmoid(w_sg . h).
     ``act``: the experts' gated activation (2 clamped GLU, 0 plain SiLU GLU: no ``limit``);
+    ``scoring``: "softmax", or "sigmoid" = every score on its own, s = sigmoid(W_r h);
     ``renorm``: the chosen scores are divided by their sum (= a softmax over the chosen logits
     alone); ``router_bias``: the router has a bias ``router.b`` that is part of the logits;
     ``correction`` False: no choice-only correction tensor.
@@ -735,8 +851,9 @@ class GroupRoutedMoE(_Block):
 
     def __init__(self, width: int, experts: int, top: int, ff: int, limit: float, groups: int, keep: int,
                  shared_ff: int, shared_limit: float, device, dtype, act: int = 2, renorm: bool = False,
-                 router_bias: bool = False, correction: bool = True):
+                 router_bias: bool = False, correction: bool = True, scoring: str = "softmax"):
         super().__init__(device, dtype)
+        self.scoring = scoring
         if groups < 1 or experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups):
             raise ValueError(f"moe: {experts} experts in {groups} groups, {keep} kept, top {top}")
         if experts > 512 or top > 16:
@@ -755,6 +872,7 @@ class GroupRoutedMoE(_Block):
         self.router_b = self._put(t["router.b"], torch.float32) if self.has_rb else None
         self.w13 = self._put(torch.stack([torch.cat([t[f"e{e}.gate"], t[f"e{e}.up"]], 0) for e in range(self.E)]))
         self.w2 = self._put(torch.stack([t[f"e{e}.down"] for e in range(self.E)]))
+        expert_layout(self)
         if self.sff:
             self.w_sgu, self.w_sd = self._put(torch.cat([t["shared.gate"], t["shared.up"]], 0)), self._put(t["shared.down"])
 
@@ -764,17 +882,18 @@ class GroupRoutedMoE(_Block):
         self.router_b = torch.zeros(self.E, dtype=torch.float32, device=self.device) if self.has_rb else None
         self.w13, self.w2 = self._rand(gen, self.E, 2 * self.ff, self.width, std=std), self._rand(
             gen, self.E, self.width, self.ff, std=std)
+        expert_layout(self)
         if self.sff:
             self.w_sgu, self.w_sd = self._rand(gen, 2 * self.sff, self.width, std=std), self._rand(
                 gen, self.width, self.sff, std=std)
 
     def grouped_ok(self, h: torch.Tensor) -> bool:
-        return h.is_cuda and h.dtype == torch.bfloat16 and self.width % 32 == 0 and self.ff % 32 == 0
+        return h.is_cuda and grouped_experts_ok(self)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         T, W = h.shape
         logits = ops.lm_head_f32(h, self.w_router)                        # fp32 [T, E (+ shared gate)]
-        tw, tid = ops.moe_route(logits[:, :self.E], self.k, self.renorm, "softmax", bias=self.correction,
+        tw, tid = ops.moe_route(logits[:, :self.E], self.k, self.renorm, self.scoring, bias=self.correction,
                                 n_group=self.groups, topk_group=self.keep, group_mode=3 if self.groups > 1 else 0,
                                 logit_bias=self.router_b)
         sh = None
@@ -786,9 +905,9 @@ class GroupRoutedMoE(_Block):
             return ops.fused_moe(h, tw, tid, self.w13, self.w2, act=self.act, limit=self.limit,
                                  add=sh.contiguous() if sh is not None else None)
         wd = torch.zeros(T, self.E, dtype=torch.float32, device=h.device).scatter_(1, tid.long(), tw)
-        gu = torch.matmul(h, self.w13.transpose(1, 2))                    # [E, T, 2 ff]
+        gu = torch.matmul(h, self.w13)                                    # [E, T, 2 ff]
         hh = ops.act_and_mul(gu.view(self.E * T, 2 * self.ff), self.act, limit=self.limit).view(self.E, T, self.ff)
-        y = (torch.bmm(hh, self.w2.transpose(1, 2)).float() * wd.t()[:, :, None]).sum(0)
+        y = (torch.bmm(hh, self.w2).float() * wd.t()[:, :, None]).sum(0)
         return (y if sh is None else y + sh.float()).to(h.dtype)
 
 

@@ -396,14 +396,15 @@ def wide_norm_rope_cache(q, k, v, positions, cos_sin, rot_dim: int, interleaved:
 def head_gate(o: torch.Tensor, g: torch.Tensor, vdim: int, kind: int = 0) -> torch.Tensor:
     """Output gate of an attention layer: ``o`` [T, H, D] (head width possibly padded beyond
     ``vdim``) times ``sigmoid(g)`` (kind 0) or ``silu(g)`` (kind 1), g a row-strided [T, H*vdim]
-    view -> contiguous [T, H*vdim] (the out-projection's input, padding dropped)."""
+    view, or [T, H]: one gate per head -> contiguous [T, H*vdim] (the out-projection's input,
+    padding dropped).  (vdim = 1: both readings of g agree.)"""
     if not _gpu(o):
         return ref.head_gate(o, g, vdim, kind)
     T, H, D = o.shape
-    assert o.is_contiguous() and g.stride(1) == 1
+    assert o.is_contiguous() and g.stride(1) == 1 and g.shape[1] in (H, H * vdim)
     out = torch.empty(T, H * vdim, dtype=o.dtype, device=o.device)
     call("ome_head_gate", o.data_ptr(), g.data_ptr(), g.stride(0), out.data_ptr(), T, H, D, vdim, int(kind),
-         _f32(o, g), stream_ptr())
+         _f32(o, g), int(g.shape[1] == H), stream_ptr())
     return out
 
 
@@ -2011,7 +2012,8 @@ def seq_rows(seqs: tuple, T: int) -> tuple[torch.Tensor, torch.Tensor]:
 
 def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim: int, interleaved: bool,
                     unit_norm: bool, eps: float, q_out, k_cache, v_cache, slots, Hq: int, Hkv: int, dim: int,
-                    vdim: int, rows: tuple | None = None) -> None:
+                    vdim: int, rows: tuple | None = None, bias: tuple | None = None, head_norm: tuple | None = None,
+                    v_mix: tuple | None = None, v_out: torch.Tensor | None = None) -> None:
     """Attention input with short causal convolutions.  q [T, Hq*dim], k [T, Hkv*dim], v [T,
     Hkv*vdim] (row-strided views of one projection) each pass a depthwise convolution over time
     (taps ``wq`` / ``wk`` / ``wv`` [channels, K], no bias, no activation; all None: no
@@ -2022,16 +2024,30 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
     D], k / v into the paged cache at ``slots`` (head tails beyond dim / vdim are zero).  ``tail``
     [slots, K-1, C] (C = all q, k, v channels, model dtype) keeps every sequence's last K-1
     projected rows; ``seqs`` = (cu, slot, reset).  Convolution, rotation and norm are fp32.
+    ``bias`` = (bq, bk, bv): added to the projections before the convolution (``tail`` holds them
+    without it; rows before a sequence's position 0 stay zero).  ``head_norm`` = (wq, wk) of width
+    ``dim``: RMS norm of every q / k head times that weight, BEFORE the rotation.  ``v_mix`` = (lam
+    fp32 [1], v_first [T, Hkv*vdim]): v <- (1 - lam) v + lam v_first, the mixed v is what is cached.
+    ``v_out`` [T, Hkv*vdim] receives the values (another layer's ``v_first``).
     ``rows`` = :func:`seq_rows` of the step (computed here when absent).  Head widths in multiples
-    of 8 with up to 6 taps and interleaved pairs run a row-parallel kernel without LDS (8 channels
-    per lane, 16-byte accesses, the tails rewritten by a second small launch); everything else the
+    of 8 with up to 6 taps and interleaved pairs (or halves of a multiple of 8) run a row-parallel
+    kernel without LDS (8 channels per lane, 16-byte accesses, the tails rewritten by a second small launch); everything else the
     tiled general kernel."""
     P, D = k_cache.shape[2], k_cache.shape[3]
     assert dim <= D and vdim <= D and rot_dim <= dim and rot_dim % 2 == 0
     if not _gpu(q):
         return ref.conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim, interleaved, unit_norm,
-                                   eps, q_out, k_cache, v_cache, slots, Hq, Hkv, dim, vdim, P)
-    f32 = _f32(q, k, v, wq, wk, wv, tail, q_out, k_cache, v_cache)
+                                   eps, q_out, k_cache, v_cache, slots, Hq, Hkv, dim, vdim, P, bias, head_norm, v_mix, v_out)
+    bq, bk, bv = bias or (None, None, None)
+    qn, kn = head_norm or (None, None)
+    lam, v_first = v_mix or (None, None)
+    f32 = _f32(q, k, v, wq, wk, wv, tail, q_out, k_cache, v_cache, bq, bk, bv, qn, kn, v_first, v_out)
+    for z, n in ((bq, Hq * dim), (bk, Hkv * dim), (bv, Hkv * vdim), (qn, dim), (kn, dim)):
+        assert z is None or (z.numel() == n and z.is_contiguous())
+    for z in (v_first, v_out):
+        assert z is None or (tuple(z.shape) == (q.shape[0], Hkv * vdim) and z.is_contiguous())
+    assert lam is None or (lam.dtype == torch.float32 and lam.numel() == 1)
+    extra = (ptr(bq), ptr(bk), ptr(bv), ptr(qn), ptr(kn), ptr(lam), ptr(v_first), ptr(v_out))
     cu, slot, reset = seqs
     K = 0 if wq is None else wq.shape[1]
     assert q_out.is_contiguous() and k_cache.is_contiguous() and v_cache.is_contiguous()
@@ -2041,14 +2057,14 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
         assert tuple(wq.shape) == (Hq * dim, K) and tuple(wk.shape) == (Hkv * dim, K) and \
             tuple(wv.shape) == (Hkv * vdim, K) and wq.is_contiguous() and wk.is_contiguous() and wv.is_contiguous()
         assert K == 1 or (tail.is_contiguous() and tuple(tail.shape[1:]) == (K - 1, (Hq + Hkv) * dim + Hkv * vdim))
-    if (interleaved or rot_dim == 0) and K <= 6 and dim % 8 == 0 and vdim % 8 == 0:
+    if (interleaved or rot_dim % 16 == 0) and K <= 6 and dim % 8 == 0 and vdim % 8 == 0:
         rs, rl = rows if rows is not None else seq_rows(seqs, q.shape[0])
         rc = load().ome_conv_rope_cache_vec(
             q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), ptr(wq), ptr(wk), ptr(wv),
             K, ptr(tail) if K > 1 else None, _i32(cu).data_ptr(), _i32(slot).data_ptr(), _i32(reset).data_ptr(),
             slot.shape[0], _i32(rs).data_ptr(), _i32(rl).data_ptr(), _i32(positions).data_ptr(), cos_sin.data_ptr(),
-            int(rot_dim), int(bool(unit_norm)), float(eps), q_out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
-            _i32(slots).data_ptr(), q.shape[0], Hq, Hkv, dim, vdim, D, P, f32, stream_ptr())
+            int(rot_dim), int(bool(interleaved)), int(bool(unit_norm)), float(eps), q_out.data_ptr(), k_cache.data_ptr(),
+            v_cache.data_ptr(), _i32(slots).data_ptr(), q.shape[0], Hq, Hkv, dim, vdim, D, P, *extra, f32, stream_ptr())
         if rc == 0:
             return
         if rc != -9:     # -9: a shape or alignment the row-parallel kernel is not built for
@@ -2057,7 +2073,64 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
          ptr(wq), ptr(wk), ptr(wv), K, ptr(tail) if K > 1 else None, _i32(cu).data_ptr(), _i32(slot).data_ptr(),
          _i32(reset).data_ptr(), slot.shape[0], _i32(positions).data_ptr(), cos_sin.data_ptr(), int(rot_dim),
          int(bool(interleaved)), int(bool(unit_norm)), float(eps), q_out.data_ptr(), k_cache.data_ptr(),
-         v_cache.data_ptr(), _i32(slots).data_ptr(), q.shape[0], Hq, Hkv, dim, vdim, D, P, f32, stream_ptr())
+         v_cache.data_ptr(), _i32(slots).data_ptr(), q.shape[0], Hq, Hkv, dim, vdim, D, P, *extra, f32, stream_ptr())
+
+
+def stream_step(y: torch.Tensor, w: torch.Tensor, groups: int, eps: float, res: torch.Tensor | None = None,
+                ids: torch.Tensor | None = None, hist: torch.Tensor | None = None, k: int = 0,
+                coef: torch.Tensor | None = None, x_out: torch.Tensor | None = None, out_dtype=None):
+    """Step of an fp32 residual stream with the norm on the sublayer's OUTPUT, in ``groups`` equal
+    consecutive parts of channels (each divided by its own root mean square), and an average over
+    depth: ``X = res + norm(y) * w`` (``res`` None: the norm alone); with ``hist`` [n, T, H] fp32
+    entry ``k`` becomes X; with ``coef`` fp32 [k+1] ``x = sum_{j<k} coef[j] hist[j] + coef[k] X``,
+    else x = X.  ``x_out`` [T, H] fp32 receives x (never ``hist``'s entry k when ``coef`` is given);
+    returns x rounded to ``out_dtype`` (the next GEMM's input), or None.  y: w's dtype or fp32; with
+    ``ids`` row t of y is ``y[ids[t]]`` (an embedding table).  All sums are fp32."""
+    if not _gpu(y):
+        return ref.stream_step(y, w, groups, eps, res, ids, hist, k, coef, x_out, out_dtype)
+    T, H = (y.shape[0] if ids is None else ids.shape[0]), y.shape[1]
+    f32 = _f32(w)
+    assert y.dim() == 2 and y.stride(1) == 1 and y.dtype in (torch.float32, w.dtype) and w.is_contiguous()
+    assert w.numel() == H and H % groups == 0
+    for t in (res, x_out):
+        assert t is None or (t.shape == (T, H) and t.dtype == torch.float32 and t.stride(1) == 1)
+    assert hist is None or (hist.dtype == torch.float32 and hist.shape[1:] == (T, H) and hist.is_contiguous() and k < hist.shape[0])
+    assert coef is None or (hist is not None and coef.dtype == torch.float32 and coef.numel() == k + 1 and coef.is_contiguous())
+    assert out_dtype is None or out_dtype == w.dtype
+    out = torch.empty(T, H, dtype=out_dtype, device=y.device) if out_dtype is not None else None
+    call("ome_stream_step", y.data_ptr(), y.stride(0), int(y.dtype == torch.float32), ptr(ids) if ids is None else
+         _i32(ids).data_ptr(), y.shape[0], ptr(res), res.stride(0) if res is not None else 0, w.data_ptr(), int(groups),
+         float(eps), ptr(hist), T * H, int(k), ptr(coef), ptr(x_out), x_out.stride(0) if x_out is not None else 0,
+         ptr(out), H, T, H, f32, stream_ptr())
+    return out
+
+
+def mingru_scan(z: torch.Tensor, x: torch.Tensor, g: torch.Tensor, zb: torch.Tensor, xb: torch.Tensor,
+                state: torch.Tensor, cu, slot, reset, single_rows: bool = False) -> torch.Tensor:
+    """minGRU core over a varlen batch: z = sigmoid(z_raw + zb), candidate c = u + 1/2 where u =
+    x_raw + xb >= 0 and sigmoid(u) elsewhere, ``S_t = S_{t-1} + z (c - S_{t-1})`` element by
+    element, returns ``S_t * silu(g)`` [T, width].  z / x / g: row-strided views of one projection;
+    ``state`` fp32 [slots, width] is continued / updated (``reset[s]``: start from zeros).  Rows of
+    a sequence are cut into chunks that run side by side (see mingru.hip); ``single_rows``: the
+    caller knows that no sequence has more than one row."""
+    T, width = z.shape
+    out = torch.empty(T, width, dtype=z.dtype, device=z.device)
+    if not _gpu(z):
+        return ref.mingru_scan(z, x, g, zb, xb, state, cu, slot, reset, out)
+    assert z.stride() == x.stride() == g.stride() and z.stride(1) == 1 and state.dtype == torch.float32
+    assert state.is_contiguous() and state.shape[1] == width and zb.numel() == xb.numel() == width
+    f32 = _f32(z, x, g, zb, xb)
+    S = slot.shape[0]
+    ch = 32 if T <= 1024 else (64 if T <= 4096 else 128)
+    if single_rows or T <= ch:
+        chunks, tmp = S, None
+    else:
+        chunks = -(-T // ch) + S
+        tmp = torch.empty(chunks, 2, width, dtype=torch.float32, device=z.device)
+    call("ome_mingru_scan", z.data_ptr(), x.data_ptr(), g.data_ptr(), z.stride(0), zb.data_ptr(), xb.data_ptr(),
+         state.data_ptr(), _i32(cu).data_ptr(), _i32(slot).data_ptr(), _i32(reset).data_ptr(), S, ptr(tmp),
+         out.data_ptr(), T, width, ch, chunks, f32, stream_ptr())
+    return out
 
 
 def talking_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,

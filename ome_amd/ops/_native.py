@@ -44,7 +44,10 @@ _SIGNATURES = {
                                      i32, i32, i32, i32, i32, i32, i32, vp, i32, vp],
         "ome_pair_embedding_f32": [vp, vp, vp, vp, vp, i32, i32, i32, f32, i32, i64, i64, vp, vp, vp, i32, i32, vp],
         "ome_diff_head_norm": [vp, vp, i32, i32, i32, i32, i32, f32, f32, f32, i32, vp],
-        "ome_head_gate": [vp, vp, i64, vp, i32, i32, i32, i32, i32, i32, vp],
+        "ome_head_gate": [vp, vp, i64, vp, i32, i32, i32, i32, i32, i32, i32, vp],
+        "ome_stream_step": [vp, i64, i32, vp, i32, vp, i64, vp, i32, f32, vp, i64, i32, vp, vp, i64, vp, i64, i32, i32,
+                            i32, vp],
+        "ome_mingru_scan": [vp, vp, vp, i64, vp, vp, vp, vp, vp, vp, i32, vp, vp, i32, i32, i32, i32, i32, vp],
         "ome_paged_attention_f32": [vp, i64, vp, vp, vp, i32, vp, vp, vp, i64, i32, i32, i32, i32, i32, f32, i32,
                                     i32, vp, vp],
         "ome_post_norm_add": [vp, i64, vp, i64, vp, vp, vp, i64, i32, i32, f32, i32, i32, vp],
@@ -63,9 +66,11 @@ _SIGNATURES = {
         "ome_shift_norm": [vp, vp, i64, vp, i64, f32, vp, i64, f32, vp, f32, vp, vp, vp, vp, vp, i32, vp, i64, i32,
                            i32, f32, i32, vp, vp],
         "ome_conv_rope_cache": [vp, i64, vp, i64, vp, i64, vp, vp, vp, i32, vp, vp, vp, vp, i32, vp, vp, i32, i32, i32,
-                                f32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, vp],
+                                f32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, vp, vp, vp, vp, vp, vp, vp, vp,
+                                i32, vp],
         "ome_conv_rope_cache_vec": [vp, i64, vp, i64, vp, i64, vp, vp, vp, i32, vp, vp, vp, vp, i32, vp, vp, vp, vp, i32,
-                                    i32, f32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, vp],
+                                    i32, i32, f32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, vp, vp, vp, vp, vp,
+                                    vp, vp, vp, i32, vp],
         "ome_talking_prefill": [vp, i64, vp, vp, vp, i32, vp, vp, vp, i32, i32, vp, i64, vp, i64, i32, i32, i32, i32,
                                 i32, f32, i32, vp, vp, vp, vp, i32, i32, vp, vp, vp],
         "ome_talking_attn": [vp, i64, vp, vp, vp, i32, vp, vp, vp, i64, vp, i64, i32, i32, i32, i32, i32, i32, f32,

@@ -341,9 +341,9 @@ def wide_norm_rope_cache(q, k, v, positions, cos_sin, rot_dim, interleaved, qn_w
 
 def head_gate(o, g, vdim: int, kind: int = 0):
     """``o`` [T, H, D] (attention output, head dim possibly padded) times ``sigmoid(g)`` (kind 0)
-    or ``silu(g)`` (kind 1), g [T, H * vdim] -> [T, H * vdim]."""
+    or ``silu(g)`` (kind 1), g [T, H * vdim] or one per head [T, H] -> [T, H * vdim]."""
     T, H, _ = o.shape
-    gf = g.float().view(T, H, vdim)
+    gf = g.float().reshape(T, H, vdim if g.shape[1] == H * vdim else 1)
     gate = torch.sigmoid(gf) if kind == 0 else torch.nn.functional.silu(gf)
     return (o[:, :, :vdim].float() * gate).reshape(T, H * vdim).to(o.dtype)
 
@@ -825,17 +825,23 @@ def shift_norm(res, w, eps, x1, s1, x2, s2, w_offset, shift, state, seqs, out_dt
 
 
 def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim, interleaved, unit_norm, eps, q_out,
-                    k_cache, v_cache, slots, Hq, Hkv, dim, vdim, P) -> None:
+                    k_cache, v_cache, slots, Hq, Hkv, dim, vdim, P, bias=None, head_norm=None, v_mix=None,
+                    v_out=None) -> None:
     """Depthwise causal convolution of q / k / v over time (taps ``w*`` [C, K], no bias, no
     activation; ``tail`` [slots, K-1, C] holds every sequence's last K-1 projected rows, C = all q,
     k, v channels), rotary embedding of q and k, then (``unit_norm``) each head divided by its root
-    mean square, q -> ``q_out`` [T, Hq, D], k / v -> paged cache."""
+    mean square, q -> ``q_out`` [T, Hq, D], k / v -> paged cache.  ``bias`` (q, k, v) before the
+    convolution, ``head_norm`` (q, k weights) before the rotation, ``v_mix`` (lam, v_first) and
+    ``v_out`` on the values."""
     T = q.shape[0]
     if T == 0:
         return
     D = k_cache.shape[3]
     x = torch.cat([q, k, v], 1).float()
-    if wq is not None:
+    b = torch.cat([t.float() for t in bias]) if bias is not None else torch.zeros(x.shape[1], device=x.device)
+    if wq is None:
+        x = x + b
+    else:
         wt = torch.cat([wq, wk, wv], 0).float()                    # [C, K]
         K = wt.shape[1]
         cu, slot, reset = seqs
@@ -852,6 +858,9 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
             else:
                 seq = x[r0:r1]
             L = r1 - r0
+            # the bias counts for the rows of the sequence, not for the zeros before its position 0
+            real = torch.arange(-(K - 1), L, device=x.device) + int(positions[r0]) >= 0
+            seq = seq + b * real[:, None]
             y[r0:r1] = sum(wt[:, j] * seq[j:j + L] for j in range(K))
         x = y
     nq, nk = Hq * dim, Hkv * dim
@@ -859,8 +868,10 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
     cs = cos_sin[positions.long()].float()
     cos, sin = cs[:, None, :half], cs[:, None, half:rot_dim]
 
-    def prep(z, H):
+    def prep(z, H, nw):
         z = z.reshape(T, H, dim).clone()
+        if nw is not None:
+            z = z * torch.rsqrt(z.pow(2).mean(-1, keepdim=True) + eps) * nw.float()
         if rot_dim > 0:
             if interleaved:
                 a, b = z[..., 0:rot_dim:2].clone(), z[..., 1:rot_dim:2].clone()
@@ -874,7 +885,14 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
             z = z * torch.rsqrt(z.pow(2).mean(-1, keepdim=True) + eps)
         return z
 
-    qf, kf = prep(x[:, :nq], Hq), prep(x[:, nq:nq + nk], Hkv)
+    qn, kn = head_norm if head_norm is not None else (None, None)
+    qf, kf = prep(x[:, :nq], Hq, qn), prep(x[:, nq:nq + nk], Hkv, kn)
+    vf = x[:, nq + nk:]
+    if v_mix is not None:
+        lam = v_mix[0].float()
+        vf = (1 - lam) * vf + lam * v_mix[1].float()
+    if v_out is not None:
+        v_out.copy_(vf)
     q_out.zero_()
     q_out[:, :, :dim] = qf.to(q_out.dtype)
     ok = slots >= 0
@@ -883,7 +901,7 @@ def conv_rope_cache(q, k, v, wq, wk, wv, tail, seqs, positions, cos_sin, rot_dim
     kp = torch.zeros(int(ok.sum()), Hkv, D, dtype=k_cache.dtype, device=k_cache.device)
     kp[:, :, :dim] = kf[ok].to(k_cache.dtype)
     vp = torch.zeros(int(ok.sum()), Hkv, D, dtype=v_cache.dtype, device=v_cache.device)
-    vp[:, :, :vdim] = x[:, nq + nk:].reshape(T, Hkv, vdim)[ok].to(v_cache.dtype)
+    vp[:, :, :vdim] = vf.reshape(T, Hkv, vdim)[ok].to(v_cache.dtype)
     k_cache[page, :, off, :] = kp
     v_cache[page, :, :, off] = vp
 
@@ -919,4 +937,38 @@ def talking_attn(q, k_cache, v_cache, block_tables, row_seq, row_pos, scale, win
         if gate is not None:
             o = o * torch.sigmoid(gate[t].float())[:, None]
         out[t] = o.reshape(-1).to(out.dtype)
+    return out
+
+
+def stream_step(y, w, groups, eps, res, ids, hist, k, coef, x_out, out_dtype):
+    yf = (y if ids is None else y[ids.long()]).float()
+    T, H = yf.shape
+    p = yf.view(T, groups, H // groups)
+    x = (p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)).view(T, H) * w.float()
+    if res is not None:
+        x = x + res
+    if hist is not None:
+        hist[k] = x
+    if coef is not None:
+        x = sum(coef[j] * hist[j] for j in range(k + 1))
+    if x_out is not None:
+        x_out.copy_(x)
+    return x.to(out_dtype) if out_dtype is not None else None
+
+
+def mingru_scan(z, x, g, zb, xb, state, cu, slot, reset, out):
+    zf = torch.sigmoid(z.float() + zb.float())
+    u = x.float() + xb.float()
+    c = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    gate = torch.nn.functional.silu(g.float())
+    for s in range(len(slot)):
+        r0, r1 = int(cu[s]), int(cu[s + 1])
+        if r1 <= r0:
+            continue
+        st = state[int(slot[s])]
+        S = torch.zeros_like(st) if int(reset[s]) else st.clone()
+        for t in range(r0, r1):
+            S = S + zf[t] * (c[t] - S)
+            out[t] = (S * gate[t]).to(out.dtype)
+        st.copy_(S)
     return out
