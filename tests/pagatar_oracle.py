@@ -225,3 +225,103 @@ def forward(cfg, weights, tokens, residuals=None, margins=None):
         if residuals is not None:
             residuals.append(x.clone())
     return group_norm(x, W["final.norm"], groups, eps) @ W["embed"].T
+
+
+# ------------------------------------------------------------------------------------ makers
+def moe(experts=5, top=2, ff=12):
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+
+
+def attn_layer(heads=4, kv_heads=2, dim=8, vdim=6, chunk=7, conv=3, rot_dims=4, base=100.0, scaling=None, scale=0.5,
+               v_mix=False, mlp=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": chunk}, "scale": scale,
+         "conv": conv, "v_mix": v_mix}
+    if rot_dims:
+        m["rot"] = {"base": base, "dims": rot_dims}
+        if scaling:
+            m["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def latent_layer(heads=3, dim=8, rot_dim=4, vdim=6, kv_rank=10, q_rank=12, base=50.0, scale=0.4, mlp=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "q_rank": q_rank, "scale": scale,
+         "rot": {"base": base, "dims": rot_dim}}
+    return {"type": "latent_attention", "mixer": m, "mlp": mlp}
+
+
+def gru_layer(inner=20, mlp=None):
+    return {"type": "mingru", "mixer": {"width": inner}, "mlp": mlp}
+
+
+def make_config(layers, width=24, vocab=41, eps=1e-5, groups=3):
+    return {"architecture": "Pagatar", "layers": layers, "norm": {"eps": eps, "groups": groups}, "vocab": vocab, "width": width}
+
+
+def make_weights(cfg, seed=0, dtype=torch.bfloat16):
+    """Random checkpoint tensors (values exactly representable in ``dtype``), sized so that the
+    stream stays O(1), scores spread over a few units and states remember a few dozen tokens."""
+    g = torch.Generator().manual_seed(seed)
+    W, V = cfg["width"], cfg["vocab"]
+
+    def rnd(*shape, s=1.0):
+        return (torch.randn(*shape, generator=g) * s).to(dtype)
+
+    def lin(o, i, gain=1.0):
+        return rnd(o, i, s=gain / math.sqrt(i))
+
+    def gain(n, at=1.0):
+        return (at + 0.2 * torch.randn(n, generator=g)).to(dtype)
+
+    t = {"embed": rnd(V, W, s=0.7), "embed.norm": gain(W), "final.norm": gain(W)}
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        t[p + "norm1"] = gain(W, 0.8)
+        if L["type"] == "attention":
+            H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            for n, c in (("q", H * d), ("k", G * d), ("v", G * dv)):
+                t[p + "mix." + n], t[p + "mix." + n + ".b"] = lin(c, W), rnd(c, s=0.5)
+                if m.get("conv"):
+                    t[p + "mix." + n + ".conv"] = rnd(c, m["conv"], s=0.6)
+            t[p + "mix.q.norm"], t[p + "mix.k.norm"] = gain(d), gain(d)
+            t[p + "mix.g"], t[p + "mix.o"] = lin(H * dv, W), lin(W, H * dv)
+            if m.get("v_mix"):
+                t[p + "mix.vmix"] = (0.3 + 0.4 * torch.rand((), generator=g)).to(dtype)
+        elif L["type"] == "latent_attention":
+            H, d, r, dv, R, Q = (m[n] for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank"))
+            t[p + "mix.dq"], t[p + "mix.dq.norm"], t[p + "mix.uq"] = lin(Q, W), gain(Q), lin(H * (d + r), Q, 1.5)
+            t[p + "mix.dkv"], t[p + "mix.dkv.norm"] = lin(R + r, W), gain(R)
+            t[p + "mix.uk"], t[p + "mix.uv"] = lin(H * d, R, 1.5), lin(H * dv, R)
+            t[p + "mix.g"], t[p + "mix.o"] = lin(H, W), lin(W, H * dv)
+        else:
+            n = m["width"]
+            t[p + "mix.z"], t[p + "mix.x"], t[p + "mix.g"] = lin(n, W), lin(n, W), lin(n, W)
+            t[p + "mix.z.b"] = (-3 + 3 * torch.rand(n, generator=g)).to(dtype)
+            t[p + "mix.x.b"], t[p + "mix.o"] = rnd(n, s=0.5), lin(W, n)
+        t[p + "dwa"] = torch.cat([rnd(i + 1, s=0.2), torch.ones(1, dtype=dtype)])
+        f = L.get("mlp")
+        if not f:
+            continue
+        E, ff = f["router"]["experts"], f["expert"]["ff"]
+        t[p + "norm2"] = gain(W, 0.8)
+        t[p + "mlp.router"], t[p + "mlp.correction"] = lin(E, W, 2.0), rnd(E, s=0.3)
+        for j in range(E):
+            t[p + f"mlp.e{j}.gate"], t[p + f"mlp.e{j}.up"], t[p + f"mlp.e{j}.down"] = lin(ff, W), lin(ff, W), lin(W, ff)
+    return t
+
+
+def write_model(folder, cfg, weights):
+    from safetensors.torch import save_file
+
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file({k: v.contiguous() for k, v in weights.items()}, os.path.join(folder, "model.safetensors"))
+    return folder
+
+
+def router_margin(cfg, weights, tokens):
+    """Smallest gap between the last chosen and the first unchosen choice score over all routed
+    evaluations of a prompt (infinite when every expert is always chosen)."""
+    m = [math.inf]
+    forward(cfg, weights, tokens, margins=m)
+    return m[0]
