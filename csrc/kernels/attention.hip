@@ -742,6 +742,10 @@ __global__ __launch_bounds__(512) void paged_prefill_kernel(
   const int win_lo = attn_lo(prefix + r0, window) & ~31;
   const int keep_end = (scl.keep + 31) & ~31;
   const int kv_lo = scl.keep > 0 ? 0 : win_lo;
+  // first visible key of this lane's two rows, and the key from which every row of the item sees all
+  // (keys at or beyond it need the mask only at the diagonal)
+  const int row_lo[2] = {attn_lo(prefix + r0 + n, window), attn_lo(prefix + r0 + 16 + n, window)};
+  const int all_lo = attn_lo(prefix + r_hi - 1, window);
   const int* bt = block_tables + (int64_t)s * bt_stride;
   const int64_t kpage = (int64_t)Hkv * P * D;
 
@@ -782,8 +786,7 @@ __global__ __launch_bounds__(512) void paged_prefill_kernel(
           sc[rb][1] = mfma16(a1, qf[rb][ks], sc[rb][1]);
         }
       }
-      const bool need_mask = (kb + 32 > prefix + r0 + 1) || (kb + 32 > kv_len) || (window > 0 || window < -1) ||
-                             scl.bs_shift != 0;
+      const bool need_mask = (kb + 32 > prefix + r0 + 1) || (kb + 32 > kv_len) || kb < all_lo || scl.bs_shift != 0;
       bf16x8 pb[2];
       float alpha[2];
 #pragma unroll
@@ -799,7 +802,7 @@ __global__ __launch_bounds__(512) void paged_prefill_kernel(
             const int key = kb + 16 * X + 4 * g + i;
             if (al != 0.f) v += al * (float)(key - qpos);
             if (need_mask) {
-              const bool ok = key <= qlim && key < kv_len && scl.in_window(key, attn_lo(qpos, window)) &&
+              const bool ok = key <= qlim && key < kv_len && scl.in_window(key, row_lo[rb]) &&
                                scl.bs_visible(qpos, key, head);
               v = ok ? v : OME_NEG_INF;
             }
@@ -932,6 +935,10 @@ __global__ __launch_bounds__(64 * NW, 8 / NW) void paged_prefill_v2_kernel(
     kv_lo = max(kv_lo, c_lo);
     kv_end = min(kv_end, c_lo + chunk);
   }
+  // first visible key of this lane's two rows, and the key from which all rows of the wave see all
+  // (keys at or beyond it need the mask only at the diagonal)
+  const int row_lo[2] = {attn_lo(prefix + r0 + n, window), attn_lo(prefix + r0 + 16 + n, window)};
+  const int all_lo = attn_lo(prefix + min(r0 + 32, q_len) - 1, window);
   const int* bt = block_tables + (int64_t)s * bt_stride;
   const int64_t kpage = (int64_t)Hkv * P * D;
 
@@ -1029,8 +1036,7 @@ __global__ __launch_bounds__(64 * NW, 8 / NW) void paged_prefill_v2_kernel(
         bf16x8 pb[2];
         float alpha[2];
         const bool need_mask =
-            (kbu + 32 > prefix + r0 + 1) || (kbu + 32 > kv_len) || (window > 0 || window < -1) ||
-            scl.bs_shift != 0;
+            (kbu + 32 > prefix + r0 + 1) || (kbu + 32 > kv_len) || kbu < all_lo || scl.bs_shift != 0;
 #pragma unroll
         for (int rb = 0; rb < 2; ++rb) {
           const int qpos = prefix + r0 + 16 * rb + n;
@@ -1044,7 +1050,7 @@ __global__ __launch_bounds__(64 * NW, 8 / NW) void paged_prefill_v2_kernel(
               const int key = kbu + 16 * X + 4 * g + i;
               if (al != 0.f) v += al * (float)(key - qpos);
               if (need_mask) {
-                const bool ok = key <= qlim && key < kv_len && scl.in_window(key, attn_lo(qpos, window)) &&
+                const bool ok = key <= qlim && key < kv_len && scl.in_window(key, row_lo[rb]) &&
                                scl.bs_visible(qpos, key, head);
                 v = ok ? v : OME_NEG_INF;
               }

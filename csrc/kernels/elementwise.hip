@@ -438,27 +438,30 @@ __global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ o,
   }
 }
 
-// bf16 rows of 8-element vectors: one per thread (vdim % 8 == 0, D % 8 == 0, 16-byte aligned rows)
+// bf16 rows of 8-element vectors, one per thread (vdim % 8 == 0, D % 8 == 0, 16-byte aligned rows);
+// a workgroup is blockDim.y rows x blockDim.x vectors
 __global__ __launch_bounds__(256) void head_gate_vec_kernel(const bf16* __restrict__ o, const bf16* __restrict__ g,
-                                                            int64_t g_stride, bf16* __restrict__ out, int H, int D,
-                                                            int vdim, int kind, int per_head, int64_t total) {
-  const int64_t v = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (v >= total) return;
-  const int nv = H * vdim / 8;
-  const int64_t t = v / nv;
-  const int i = (int)(v - t * nv) * 8;
+                                                            int64_t g_stride, bf16* __restrict__ out, int T, int H,
+                                                            int D, int vdim, int kind, int per_head) {
+  const int64_t t = (int64_t)blockIdx.y * blockDim.y + threadIdx.y;
+  const int i = (blockIdx.x * blockDim.x + threadIdx.x) * 8;
+  if (t >= T || i >= H * vdim) return;
   const int h = i / vdim, d = i - h * vdim;
   const bf16x8 x = ld8(o + (t * H + h) * D + d);
-  bf16x8 gv = {};
-  float g1 = 0.f;
-  if (per_head) g1 = (float)g[t * g_stride + h];
-  else gv = ld8(g + t * g_stride + i);
   bf16x8 r;
+  if (per_head) {
+    const float z = (float)g[t * g_stride + h];
+    const float sg = __builtin_amdgcn_rcpf(1.f + __expf(-z)), m = kind == 0 ? sg : z * sg;
 #pragma unroll
-  for (int e = 0; e < 8; ++e) {
-    const float z = per_head ? g1 : (float)gv[e];
-    const float sg = 1.f / (1.f + expf(-z));
-    r[e] = (bf16)((float)x[e] * (kind == 0 ? sg : z * sg));
+    for (int e = 0; e < 8; ++e) r[e] = (bf16)((float)x[e] * m);
+  } else {
+    const bf16x8 gv = ld8(g + t * g_stride + i);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float z = (float)gv[e];
+      const float sg = __builtin_amdgcn_rcpf(1.f + __expf(-z));
+      r[e] = (bf16)((float)x[e] * (kind == 0 ? sg : z * sg));
+    }
   }
   st8(out + t * H * vdim + i, r);
 }
@@ -470,9 +473,17 @@ OME_API int ome_head_gate(const void* o, const void* g, int64_t g_stride, void* 
   const bool al = (((uintptr_t)o | (uintptr_t)out) & 15) == 0 &&
                   (per_head || (((uintptr_t)g & 15) == 0 && g_stride % 8 == 0));
   if (!f32 && vdim % 8 == 0 && D % 8 == 0 && al) {
-    const int64_t total = (int64_t)T * (H * vdim / 8);
-    head_gate_vec_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(
-        (const bf16*)o, (const bf16*)g, g_stride, (bf16*)out, H, D, vdim, kind, per_head, total);
+    const int nv = H * vdim / 8;
+    int bx = 8;
+    while (bx < nv && bx < 256) bx *= 2;
+    const int by = 256 / bx;
+    for (int t0 = 0; t0 < T; t0 += 65535 * by) {   // (grid.y holds at most 65535 blocks)
+      const int n = T - t0 < 65535 * by ? T - t0 : 65535 * by;
+      const int64_t r = t0;
+      head_gate_vec_kernel<<<dim3((nv + bx - 1) / bx, (n + by - 1) / by), dim3(bx, by), 0, stream>>>(
+          (const bf16*)o + r * H * D, (const bf16*)g + r * g_stride, g_stride, (bf16*)out + r * H * vdim, n, H, D, vdim,
+          kind, per_head);
+    }
   } else if (f32) {
     head_gate_kernel<float><<<T, 256, 0, stream>>>((const float*)o, (const float*)g, g_stride, (float*)out, H, D, vdim,
                                                    kind, per_head);

@@ -18,39 +18,55 @@
 
 namespace {
 
+// V neighbouring channels of a thread
 template <int V>
 struct Vec {
   float f[V];
 };
+// the same as they lie in memory (kept unconverted while a load is in flight)
+template <typename T, int V>
+struct Raw {
+  typedef T type __attribute__((ext_vector_type(V)));
+};
+template <typename T>
+struct Raw<T, 1> {
+  typedef T type;
+};
+template <typename T, int V>
+using raw_t = typename Raw<T, V>::type;
 
 template <typename T, int V>
-__device__ __forceinline__ Vec<V> ldv(const T* p) {
+__device__ __forceinline__ raw_t<T, V> ldr(const T* p) {
+  return *reinterpret_cast<const raw_t<T, V>*>(p);
+}
+template <typename T, int V>
+__device__ __forceinline__ Vec<V> widen(raw_t<T, V> t) {
   Vec<V> r;
   if constexpr (V == 1) {
-    r.f[0] = (float)p[0];
-  } else if constexpr (sizeof(T) == 2) {
-    const bf16x2 t = *reinterpret_cast<const bf16x2*>(p);
-    r.f[0] = (float)t[0];
-    r.f[1] = (float)t[1];
+    r.f[0] = (float)t;
   } else {
-    const float2 t = *reinterpret_cast<const float2*>(p);
-    r.f[0] = t.x;
-    r.f[1] = t.y;
+#pragma unroll
+    for (int i = 0; i < V; ++i) r.f[i] = (float)t[i];
   }
   return r;
 }
 template <typename T, int V>
+__device__ __forceinline__ Vec<V> ldv(const T* p) {
+  return widen<T, V>(ldr<T, V>(p));
+}
+template <typename T, int V>
 __device__ __forceinline__ void stv(T* p, const Vec<V>& v) {
+  raw_t<T, V> t;
   if constexpr (V == 1) {
-    p[0] = (T)v.f[0];
-  } else if constexpr (sizeof(T) == 2) {
-    *reinterpret_cast<bf16x2*>(p) = bf16x2{(bf16)v.f[0], (bf16)v.f[1]};
+    t = (T)v.f[0];
   } else {
-    *reinterpret_cast<float2*>(p) = make_float2(v.f[0], v.f[1]);
+#pragma unroll
+    for (int i = 0; i < V; ++i) t[i] = (T)v.f[i];
   }
+  *reinterpret_cast<raw_t<T, V>*>(p) = t;
 }
 
-__device__ __forceinline__ float sig(float x) { return 1.f / (1.f + __expf(-x)); }
+__device__ __forceinline__ float sig(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
 // workgroup row `z` of the grid -> (sequence, chunk of it); every wave scans the sequence lengths
 __device__ __forceinline__ bool find_chunk(const int* __restrict__ cu, int S, int CH, int z, int& s, int& c) {
@@ -78,7 +94,25 @@ __device__ __forceinline__ bool find_chunk(const int* __restrict__ cu, int S, in
   return false;
 }
 
+constexpr int64_t V4_MIN = 256 * 1024;
 constexpr int RB = 8;   // rows whose loads are in flight together
+
+template <typename T, int V, bool OUT>
+struct Batch {
+  raw_t<T, V> z[RB], x[RB], g[OUT ? RB : 1];
+};
+
+template <typename T, int V, bool OUT>
+__device__ __forceinline__ void fetch(Batch<T, V, OUT>& b, const T* __restrict__ zr, const T* __restrict__ xr,
+                                      const T* __restrict__ gr, int64_t stride, int t0, int e, int ch) {
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    const int64_t o = (int64_t)min(t0 + r, e - 1) * stride + ch;
+    b.z[r] = ldr<T, V>(zr + o);
+    b.x[r] = ldr<T, V>(xr + o);
+    if constexpr (OUT) b.g[r] = ldr<T, V>(gr + o);
+  }
+}
 
 // rows [a, e): advance S; OUT: write the gated output, otherwise gather A = prod(1 - z)
 template <typename T, int V, bool OUT>
@@ -86,25 +120,21 @@ __device__ __forceinline__ void run_rows(const T* __restrict__ zr, const T* __re
                                          int64_t stride, T* __restrict__ out, int width, int a, int e, int ch,
                                          const Vec<V>& bz, const Vec<V>& bx, Vec<V>& S, Vec<V>& A) {
   for (int t0 = a; t0 < e; t0 += RB) {
-    Vec<V> z[RB], x[RB], g[RB];
-#pragma unroll
-    for (int r = 0; r < RB; ++r) {
-      const int64_t o = (int64_t)min(t0 + r, e - 1) * stride + ch;
-      z[r] = ldv<T, V>(zr + o);
-      x[r] = ldv<T, V>(xr + o);
-      if constexpr (OUT) g[r] = ldv<T, V>(gr + o);
-    }
+    Batch<T, V, OUT> cur;
+    fetch(cur, zr, xr, gr, stride, t0, e, ch);
 #pragma unroll
     for (int r = 0; r < RB; ++r) {
       if (t0 + r >= e) break;
+      const Vec<V> z = widen<T, V>(cur.z[r]), x = widen<T, V>(cur.x[r]);
       Vec<V> y;
+      if constexpr (OUT) y = widen<T, V>(cur.g[r]);
 #pragma unroll
       for (int i = 0; i < V; ++i) {
-        const float zz = sig(z[r].f[i] + bz.f[i]);
-        const float u = x[r].f[i] + bx.f[i];
+        const float zz = sig(z.f[i] + bz.f[i]);
+        const float u = x.f[i] + bx.f[i];
         const float c = u >= 0.f ? u + 0.5f : sig(u);
         S.f[i] += zz * (c - S.f[i]);
-        if constexpr (OUT) y.f[i] = S.f[i] * g[r].f[i] * sig(g[r].f[i]);
+        if constexpr (OUT) y.f[i] = S.f[i] * y.f[i] * sig(y.f[i]);
         else A.f[i] *= 1.f - zz;
       }
       if constexpr (OUT) stv<T, V>(out + (int64_t)(t0 + r) * width + ch, y);
@@ -188,12 +218,17 @@ OME_API int ome_mingru_scan(const void* z, const void* x, const void* g, int64_t
   if (width <= 0 || CH <= 0 || chunks <= 0) return -2;
   if (chunks > 65535) return -3;
   const int esz = f32 ? 4 : 2;
-  auto al = [&](const void* p) { return ((uintptr_t)p & (2 * esz - 1)) == 0; };
-  const bool v2 = width % 2 == 0 && stride % 2 == 0 && al(z) && al(x) && al(g) && al(zb) && al(xb) && al(out) &&
-                  ((uintptr_t)state & 7) == 0 && ((uintptr_t)sum & 7) == 0;
+  // channels per thread: as wide as the alignment allows (v: 2 or 4)
+  auto ok = [&](int v) {
+    auto al = [&](const void* p) { return ((uintptr_t)p & (v * esz - 1)) == 0; };
+    return width % v == 0 && stride % v == 0 && al(z) && al(x) && al(g) && al(zb) && al(xb) && al(out) &&
+           ((uintptr_t)state & (4 * v - 1)) == 0 && ((uintptr_t)sum & (4 * v - 1)) == 0;
+  };
 #define MG(TT, VV) \
   launch<TT, VV>(z, x, g, stride, zb, xb, state, cu, slot, reset, S, sum, out, T, width, CH, chunks, stream)
-  if (f32) return v2 ? MG(float, 2) : MG(float, 1);
-  return v2 ? MG(bf16, 2) : MG(bf16, 1);
+  // (four per thread only where that still leaves a workgroup for every CU)
+  if (f32) return ok(2) ? MG(float, 2) : MG(float, 1);
+  if (ok(4) && (int64_t)chunks * width >= V4_MIN) return MG(bf16, 4);
+  return ok(2) ? MG(bf16, 2) : MG(bf16, 1);
 #undef MG
 }

@@ -1,5 +1,10 @@
 """Layer-list designs beside their closest existing model at equal size (``bench.py --arch-compare
-[--arch-design zavilorn|metitar|milenex|nivasun]``).
+[--arch-design zavilorn|metitar|milenex|nivasun|pagatar]``).
+
+Pagatar (chunked attention behind short convolutions with value mixing, minGRU, full latent attention,
+sigmoid-routed SiLU-GLU experts, output norms in channel groups and a learned average over depth)
+stands beside the same GPT-OSS-style stack of the same width, depth, head counts, mask size and expert
+sizes.
 
 Nivasun (parallel blocks: one norm feeding a mixer -- differential, key-valued or windowed latent
 attention behind a short convolution -- and a biased-router mixture of SiLU-GLU experts with a gated
@@ -143,6 +148,22 @@ def nivasun_config(s: dict, window: int = 1024) -> dict:
     return {"architecture": "Nivasun", "layers": [dif, key, dif, lat] * 2, "norm": {"eps": 1e-6}, "vocab": s["vocab"],
             "width": s["width"], "max_positions": 8192, "canon": {"taps": 4}, "logit_softcap": 25.0,
             "embedding": {"scale": 1.0, "bigram": {"buckets": 65521, "mul_prev": 36313, "mul_cur": 27191}}}
+
+
+def pagatar_config(s: dict, chunk: int = 1024) -> dict:
+    """[chunked attention, minGRU, latent attention, chunked attention] x 2 with 128-wide heads, a
+    256 + 64-wide latent row, minGRU of the model's width, every layer with 32 experts, top 4."""
+    moe = {"kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}, "expert": {"ff": s["eff"]}}
+    att = {"type": "attention", "mlp": moe,
+           "mixer": {"heads": s["heads"], "kv_heads": s["kv"], "dim": 128, "vdim": 128, "mask": {"size": chunk}, "conv": 4,
+                     "rot": {"base": 500000.0, "dims": 128, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}},
+                     "scale": 128 ** -0.5, "v_mix": True}}
+    gru = {"type": "mingru", "mlp": moe, "mixer": {"width": s["width"]}}
+    lat = {"type": "latent_attention", "mlp": moe,
+           "mixer": {"heads": s["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 256, "q_rank": 768,
+                     "scale": 192 ** -0.5, "rot": {"base": 500000.0, "dims": 64}}}
+    return {"architecture": "Pagatar", "layers": [att, gru, lat, att] * 2, "norm": {"eps": 1e-6, "groups": 4}, "vocab": s["vocab"],
+            "width": s["width"], "max_positions": 8192}
 
 
 def gpt_oss_like_config(s: dict, window: int = 1024) -> dict:
@@ -691,8 +712,165 @@ def kernel_table_nivasun(T: int = 4096, B: int = 64, ctx: int = 4096, width: int
     return rows
 
 
+def kernel_table_pagatar(T: int = 4096, B: int = 64, ctx: int = 4096, width: int = 4096) -> list[dict]:
+    """Pagatar's kernels beside their like kernels (same columns as :func:`kernel_table`)."""
+    from ome_amd import ops
+    from ome_amd.models.config import plain_rope_table
+    from ome_amd.models.mixers import GroupRoutedMoE
+
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+
+    def pair(name, new, like, bytes_new, bytes_like, note="", iters=30):
+        tn, tl = _time_us(new, iters), _time_us(like, iters)
+        fn, fl = bytes_new / tn / 1e3 / HBM_GBS, bytes_like / tl / 1e3 / HBM_GBS
+        rows.append({"kernel": name, "us": round(tn, 1), "roofline": round(fn, 3), "like_us": round(tl, 1),
+                     "like_roofline": round(fl, 3), "vs_like": round(fl / max(fn, 1e-9), 2), "note": note})
+
+    def seqs(lens):
+        cu = torch.tensor([0] + torch.tensor(lens).cumsum(0).tolist(), dtype=torch.int32, device=dev)
+        n = len(lens)
+        return cu, torch.arange(n, dtype=torch.int32, device=dev), torch.zeros(n, dtype=torch.int32, device=dev)
+
+    torch.manual_seed(0)
+    Hq, Hkv, D, P, W, L = 32, 8, 128, 16, 1024, 8
+    for R, tag, lens in ((T, "prefill", [T // 2] * 2), (B, "decode", [1] * B)):
+        sq = seqs(lens)
+        # ---- stream steps vs add + RMSNorm on a bf16 stream
+        res = torch.randn(R, width, device=dev)
+        y = torch.randn(R, width, device=dev).to(bf)
+        w = torch.ones(width, device=dev, dtype=bf)
+        rb, xb = res.to(bf), y.clone()
+        hist, x = torch.randn(L + 1, R, width, device=dev), torch.empty(R, width, device=dev)
+        like = lambda: ops.fused_add_rmsnorm(xb, rb, w, 1e-6)   # noqa: E731
+        V = 32768
+        ids, emb = torch.randint(0, V, (R,), dtype=torch.int32, device=dev), torch.randn(V, width, device=dev).to(bf)
+        pair(f"stream_step: embedding + norm in 4 groups ({tag})",
+             lambda: ops.stream_step(emb, w, 4, 1e-6, ids=ids, hist=hist, k=0, out_dtype=bf), lambda: ops.embedding(ids, emb),
+             R * width * 8, R * width * 4, "like: the plain embedding gather")
+        pair(f"stream_step: sum after a mixer ({tag})",
+             lambda: ops.stream_step(y, w, 4, 1e-6, res=res, x_out=x, out_dtype=bf), like, R * width * 12, R * width * 8,
+             "fp32 stream out of place: 12 B / element against 8")
+        coef = torch.full((L + 1,), 0.1, device=dev)
+        pair(f"stream_step: layer result + average over 8 earlier ones ({tag})",
+             lambda: ops.stream_step(y, w, 4, 1e-6, res=res, hist=hist, k=L, coef=coef, x_out=x, out_dtype=bf), like,
+             R * width * (16 + 4 * L), R * width * 8, "16 B / element + 4 per earlier result")
+        # ---- minGRU vs HGRN2's scan (matrix state) as the like recurrence
+        p = torch.randn(R, 3 * width, device=dev).to(bf)
+        zb = torch.zeros(width, device=dev, dtype=bf)
+        st = torch.zeros(len(lens), width, device=dev)
+        n = width
+        hp = torch.randn(R, 3 * n, device=dev).to(bf)
+        hst, hw = torch.zeros(len(lens), n // 128, 128, 128, device=dev), torch.ones(128, device=dev, dtype=bf)
+        gru = lambda: ops.mingru_scan(p[:, :n], p[:, n:2 * n], p[:, 2 * n:], zb, zb, st, *sq, single_rows=R == len(lens))   # noqa: E731
+        wc, stc = (torch.randn(n, 4, device=dev) * 0.3).to(bf), torch.zeros(len(lens), n, 3, device=dev, dtype=bf)
+        pair(f"mingru_scan, {width} channels ({tag}), like: conv + SiLU with a per-channel state", gru,
+             lambda: ops.ssm_conv1d(y, wc, None, stc, *sq), R * n * 8 + len(lens) * n * 8, R * n * 4 + len(lens) * n * 12,
+             "the other element-wise stateful kernel (Mamba-2 / delta-rule inputs)")
+        pair(f"mingru_scan, {width} channels ({tag}), like: HGRN2's scan", gru,
+             lambda: ops.hgrn2_scan(hp[:, :n], hp[:, n:2 * n], hp[:, 2 * n:], zb, zb, hw, hst, *sq, n // 128, 128, 128, 1e-6),
+             R * n * 8 + len(lens) * n * 8, R * n * 8 + len(lens) * n * 128 * 8,
+             "two launches per prompt step (chunk summaries, then the rows); like: a matrix state per head, 128 times the bytes")
+        # ---- attention input: convolution, biases, head norms, rotary halves, value mix vs Milenex's
+        n_pages = R // P + 2
+        kc = torch.zeros(n_pages, Hkv, P, D, device=dev, dtype=bf)
+        vc = torch.zeros(n_pages, Hkv, D, P, device=dev, dtype=bf)
+        C = (Hq + 2 * Hkv) * D
+        qkv = torch.randn(R, C, device=dev).to(bf)
+        pos = torch.arange(R, dtype=torch.int32, device=dev) % 2048
+        slots = torch.arange(R, dtype=torch.int32, device=dev) + P
+        cs = plain_rope_table(10000.0, 128, 2049, dev)
+        cs64 = plain_rope_table(10000.0, 64, 2049, dev)
+        qo = torch.empty(R, Hq, D, device=dev, dtype=bf)
+        cw = [(torch.randn(c, 4, device=dev) * 0.3).to(bf) for c in (Hq * D, Hkv * D, Hkv * D)]
+        bias = tuple(torch.randn(c, device=dev).to(bf) for c in (Hq * D, Hkv * D, Hkv * D))
+        tail = torch.zeros(len(lens), 3, C, device=dev, dtype=bf)
+        hn = torch.ones(D, device=dev, dtype=bf)
+        lam, vf = torch.full((1,), 0.3, device=dev), torch.randn(R, Hkv * D, device=dev).to(bf)
+        srows = ops.seq_rows(sq, R)
+        qv, kv_, vv = qkv[:, :Hq * D], qkv[:, Hq * D:(Hq + Hkv) * D], qkv[:, (Hq + Hkv) * D:]
+        pair(f"conv_rope_cache with biases, head norms, halves, value mix ({tag})",
+             lambda: ops.conv_rope_cache(qv, kv_, vv, *cw, tail, sq, pos, cs, 128, False, False, 1e-6, qo, kc, vc, slots, Hq, Hkv,
+                                         D, D, rows=srows, bias=bias, head_norm=(hn, hn), v_mix=(lam, vf)),
+             lambda: ops.conv_rope_cache(qv, kv_, vv, *cw, tail, sq, pos, cs64, 64, True, True, 1e-6, qo, kc, vc, slots, Hq, Hkv,
+                                         D, D, rows=srows), R * (2 * C + Hkv * D) * 2, R * C * 2 * 2,
+             "like: Milenex's use of it (unit norms, interleaved pairs)")
+        # ---- output gates
+        o = torch.randn(R, Hq, D, device=dev).to(bf)
+        g1, gf = torch.randn(R, Hq, device=dev).to(bf), torch.randn(R, Hq * D, device=dev).to(bf)
+        pair(f"head_gate, one gate per head ({tag})", lambda: ops.head_gate(o, g1, D, 0), lambda: ops.head_gate(o, gf, D, 0),
+             R * Hq * D * 4, R * Hq * D * 6, "like: the element-wise gate")
+        # ---- routed feed-forward
+        E, k, ff = 32, 4, 2048
+        moe = GroupRoutedMoE(width, E, k, ff, 0.0, 1, 1, 0, 0.0, dev, bf, act=0, scoring="sigmoid")
+        moe.init_random(torch.Generator(device=dev).manual_seed(1), 0.02)
+        xx = torch.randn(R, width, device=dev).to(bf)
+        tw, tid = ops.moe_route(torch.randn(R, E, device=dev), k, True, "softmax")
+        touched = min(E, R * k) * 3 * ff * width * 2
+        pair(f"sigmoid-routed moe 32 experts top 4 ({tag})", lambda: moe.forward(xx),
+             lambda: ops.fused_moe(xx, tw, tid, moe.w13, moe.w2, 2, 1.0), touched, touched,
+             "new: router GEMM + route + grouped GEMMs + combine; like: grouped GEMMs + combine", 10)
+    # ---- chunked attention vs the sliding window: decode (the last row of a chunk: all its keys) and prefill
+    per = ctx // P
+    kc = (torch.randn(B * per + 1, Hkv, P, D, device=dev) * 0.3).to(bf)
+    vc = (torch.randn(B * per + 1, Hkv, D, P, device=dev) * 0.3).to(bf)
+    bt = (torch.arange(B * per, dtype=torch.int32, device=dev) + 1).view(B, per)
+    sl = torch.full((B,), ctx, dtype=torch.int32, device=dev)
+    q = (torch.randn(B, Hq, D, device=dev) * 0.3).to(bf)
+    ws = ops.DecodeWorkspace(B, Hq, D, ctx, 0, dev, parts=4)
+    kvb = B * Hkv * D * 2 * 2 * W
+    pair("chunked attention decode 64 x 4096 ctx, chunks of 1024", lambda: ops.paged_decode(q, kc, vc, bt, sl, 0.09, ws, -W),
+         lambda: ops.paged_decode(q, kc, vc, bt, sl, 0.09, ws, W), kvb, kvb, "like: the sliding window of 1024", 10)
+    q_lens = [2048, 2048]
+    Tq = sum(q_lens)
+    qp = (torch.randn(Tq, Hq, D, device=dev) * 0.3).to(bf)
+    cu = torch.tensor([0, 2048, 4096], dtype=torch.int32, device=dev)
+    kl = torch.tensor(q_lens, dtype=torch.int32, device=dev)
+    bt2 = (torch.arange(2 * 128, dtype=torch.int32, device=dev) + 1).view(2, 128)
+    items = torch.tensor(ops.prefill_work_items(q_lens, q_lens), dtype=torch.int32, device=dev)
+    fc = 4.0 * Hq * D * sum(i % W + 1 for i in range(2048)) * 2
+    fw = 4.0 * Hq * D * sum(min(W, i + 1) for i in range(2048)) * 2
+    tn = _time_us(lambda: ops.paged_prefill(qp, kc, vc, bt2, cu, kl, items, 0.09, -W), 10)
+    tl = _time_us(lambda: ops.paged_prefill(qp, kc, vc, bt2, cu, kl, items, 0.09, W), 10)
+    rows.append({"kernel": "chunked attention prefill 2 x 2048 rows, chunks of 1024", "us": round(tn, 1),
+                 "roofline": round(fc / tn / 1e6 / 2.5e3, 3), "like_us": round(tl, 1),
+                 "like_roofline": round(fw / tl / 1e6 / 2.5e3, 3), "vs_like": round((fw / tl) / (fc / tn), 2),
+                 "note": "share of 2.5 PFLOP/s bf16; like: the sliding window of 1024 (more keys per row)"})
+    # ---- latent attention 256 + 64 vs the 256 + 32 row of the DeepSeek-style stack, same kernel
+    res2 = {}
+    for lat, rope in ((256, 64), (256, 32)):
+        DK, DV = ops.latent_shape(lat, rope)
+        lc = (torch.randn(B * per + 1, P, DK, device=dev) * 0.3).to(bf)
+        ql, qlp = ((torch.randn(n, Hq, DK, device=dev) * 0.3).to(bf) for n in (B, Tq))
+        mws = ops.MLAWorkspace(dev)
+        ri = torch.arange(B, dtype=torch.int32, device=dev)
+        tok_row = torch.arange(Tq, dtype=torch.int32, device=dev) // 2048
+        lens_p = (torch.arange(Tq, dtype=torch.int32, device=dev) % 2048) + 1
+        fl = 2.0 * Hq * (DK + DV) * sum(i + 1 for i in range(2048)) * 2
+        td = _time_us(lambda: ops.latent_attn(ql, lc, bt, ri, sl, 0.09, DV, mws), 10)
+        tp = _time_us(lambda: ops.latent_attn(qlp, lc, bt2, tok_row, lens_p, 0.09, DV, mws), 5)
+        res2[rope] = (td, B * ctx * DK * 2 / td / 1e3 / HBM_GBS, tp, fl / tp / 1e6 / 2.5e3)
+    for name, i in (("latent attention decode 64 x 4096 ctx, 32 heads, 320-wide rows", 0),
+                    ("latent attention prefill 2 x 2048 rows, 32 heads, 320-wide rows", 2)):
+        (tn, fn), (tl, fl_) = res2[64][i:i + 2], res2[32][i:i + 2]
+        rows.append({"kernel": name, "us": round(tn, 1), "roofline": round(fn, 3), "like_us": round(tl, 1),
+                     "like_roofline": round(fl_, 3), "vs_like": round(fl_ / fn, 2),
+                     "note": "like: the same kernel on 288-wide rows"})
+    return rows
+
+
 def run(sizes=("2k", "4k"), kernels: bool = True, only: str | None = None, design: str = "zavilorn") -> dict:
     out = {"throughput": [], "kernels": []}
+    if design == "pagatar":
+        for k in sizes:
+            s = X_SIZES[k]
+            if only in (None, "pagatar"):
+                out["throughput"].append(throughput(f"pagatar-{k}", pagatar_config(s)))
+            if only in (None, "gpt-oss"):
+                out["throughput"].append(throughput(f"gpt-oss-like-{k}", gpt_oss_like_config(s)))
+        if kernels:
+            out["kernels"] = kernel_table_pagatar()
+        return out
     if design == "nivasun":
         for k in sizes:
             s = X_SIZES[k]
@@ -740,10 +918,10 @@ def main(argv=None) -> int:
     ap = argparse.ArgumentParser(description=__doc__)
     ap.add_argument("--sizes", default="2k,4k")
     ap.add_argument("--no-kernels", action="store_true")
-    ap.add_argument("--only", choices=["zavilorn", "nemotron", "metitar", "deepseek", "milenex", "gpt-oss", "nivasun"],
+    ap.add_argument("--only", choices=["zavilorn", "nemotron", "metitar", "deepseek", "milenex", "gpt-oss", "nivasun", "pagatar"],
                     default=None,
                     help="one stack (for kernel traces)")
-    ap.add_argument("--design", choices=["zavilorn", "metitar", "milenex", "nivasun"], default="zavilorn")
+    ap.add_argument("--design", choices=["zavilorn", "metitar", "milenex", "nivasun", "pagatar"], default="zavilorn")
     ap.add_argument("--no-throughput", action="store_true", help="the kernel table only")
     a = ap.parse_args(argv)
     res = run(() if a.no_throughput else tuple(a.sizes.split(",")), not a.no_kernels, a.only, a.design)

@@ -2106,13 +2106,14 @@ def stream_step(y: torch.Tensor, w: torch.Tensor, groups: int, eps: float, res: 
 
 
 def mingru_scan(z: torch.Tensor, x: torch.Tensor, g: torch.Tensor, zb: torch.Tensor, xb: torch.Tensor,
-                state: torch.Tensor, cu, slot, reset, single_rows: bool = False) -> torch.Tensor:
+                state: torch.Tensor, cu, slot, reset, single_rows: bool = False,
+                chunk: int | None = None) -> torch.Tensor:
     """minGRU core over a varlen batch: z = sigmoid(z_raw + zb), candidate c = u + 1/2 where u =
     x_raw + xb >= 0 and sigmoid(u) elsewhere, ``S_t = S_{t-1} + z (c - S_{t-1})`` element by
     element, returns ``S_t * silu(g)`` [T, width].  z / x / g: row-strided views of one projection;
     ``state`` fp32 [slots, width] is continued / updated (``reset[s]``: start from zeros).  Rows of
     a sequence are cut into chunks that run side by side (see mingru.hip); ``single_rows``: the
-    caller knows that no sequence has more than one row."""
+    caller knows that no sequence has more than one row; ``chunk``: rows per chunk (default by T)."""
     T, width = z.shape
     out = torch.empty(T, width, dtype=z.dtype, device=z.device)
     if not _gpu(z):
@@ -2121,7 +2122,7 @@ def mingru_scan(z: torch.Tensor, x: torch.Tensor, g: torch.Tensor, zb: torch.Ten
     assert state.is_contiguous() and state.shape[1] == width and zb.numel() == xb.numel() == width
     f32 = _f32(z, x, g, zb, xb)
     S = slot.shape[0]
-    ch = 32 if T <= 1024 else (64 if T <= 4096 else 128)
+    ch = chunk or (32 if T <= 4096 else (64 if T <= 12288 else 128))
     if single_rows or T <= ch:
         chunks, tmp = S, None
     else:
