@@ -156,12 +156,12 @@ def pagatar_config(s: dict, chunk: int = 1024) -> dict:
     moe = {"kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}, "expert": {"ff": s["eff"]}}
     att = {"type": "attention", "mlp": moe,
            "mixer": {"heads": s["heads"], "kv_heads": s["kv"], "dim": 128, "vdim": 128, "mask": {"size": chunk}, "conv": 4,
-                     "rot": {"base": 500000.0, "dims": 128, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}},
+                     "rot": {"base": 10000.0, "dims": 128, "scaling": {"factor": 8.0, "original": 2048, "fast": 32.0, "slow": 1.0}},
                      "scale": 128 ** -0.5, "v_mix": True}}
     gru = {"type": "mingru", "mlp": moe, "mixer": {"width": s["width"]}}
     lat = {"type": "latent_attention", "mlp": moe,
            "mixer": {"heads": s["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 256, "q_rank": 768,
-                     "scale": 192 ** -0.5, "rot": {"base": 500000.0, "dims": 64}}}
+                     "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}}
     return {"architecture": "Pagatar", "layers": [att, gru, lat, att] * 2, "norm": {"eps": 1e-6, "groups": 4}, "vocab": s["vocab"],
             "width": s["width"], "max_positions": 8192}
 

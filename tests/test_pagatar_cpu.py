@@ -85,10 +85,10 @@ def test_chunk_edge():
 
 def test_far_key_and_page_borders():
     for j in (131, 128, 127, 112, 0):                              # keys of row 431, one long chunk / the latent layer
-        pc.planted_case(DEV, DT, "attention", 432, 431, j, [400] + [1] * 32, chunk=1000, other_chunk=200)
+        pc.planted_case(DEV, DT, "attention", 432, 431, j, [400] + [1] * 32, chunk=1000, other_chunk=210)
         pc.planted_case(DEV, DT, "latent_attention", 432, 431, j, [400] + [1] * 32)
     pc.planted_case(DEV, DT, "latent_attention", 432, 431, 16, pc.portions(432, [64, 35, 2, 17]))
-    pc.planted_case(DEV, DT, "attention", 432, 431, 400, pc.portions(432, [64, 35, 2, 17]), chunk=200, other_chunk=401)
+    pc.planted_case(DEV, DT, "attention", 432, 431, 400, pc.portions(432, [64, 35, 2, 17]), chunk=192, other_chunk=401)
 
 
 # ------------------------------------------------------------------------------ whole models

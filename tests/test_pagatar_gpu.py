@@ -60,7 +60,7 @@ def test_mingru_many_sequences():
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("T,H,D,vdim", [(5, 3, 64, 10), (4, 8, 64, 48), (33, 32, 128, 128), (2, 1, 64, 1), (3, 5, 256, 200), (9, 16, 64, 64)])
+@pytest.mark.parametrize("T,H,D,vdim", [(5, 3, 64, 10), (4, 6, 64, 56), (33, 32, 128, 128), (2, 1, 64, 1), (3, 5, 256, 200), (9, 16, 64, 64)])
 def test_head_gate_kernel(dt, T, H, D, vdim):
     pc.head_gate_case(DEV, dt, T=T, H=H, D=D, vdim=vdim)
 
@@ -164,10 +164,10 @@ def test_chunk_edge(dt):
 @pytest.mark.parametrize("dt", DTYPES)
 def test_far_key_and_page_borders(dt):
     for j in (131, 128, 127, 112, 0):
-        pc.planted_case(DEV, dt, "attention", 432, 431, j, [400] + [1] * 32, chunk=1000, other_chunk=200)
+        pc.planted_case(DEV, dt, "attention", 432, 431, j, [400] + [1] * 32, chunk=1000, other_chunk=210)
         pc.planted_case(DEV, dt, "latent_attention", 432, 431, j, [400] + [1] * 32)
     pc.planted_case(DEV, dt, "latent_attention", 432, 431, 16, pc.portions(432, [64, 35, 2, 17]))
-    pc.planted_case(DEV, dt, "attention", 432, 431, 400, pc.portions(432, [64, 35, 2, 17]), chunk=200, other_chunk=401)
+    pc.planted_case(DEV, dt, "attention", 432, 431, 400, pc.portions(432, [64, 35, 2, 17]), chunk=192, other_chunk=401)
 
 
 # ------------------------------------------------------------------------------ whole models
