@@ -27,7 +27,8 @@
 // chosen on score + bias (``e_score_correction_bias``) restricted to the best ``topk_group``
 // groups (other experts score 0, as in the HF reference); weights are the unbiased scores.
 // 3 = group score = max like 1, but experts outside the chosen groups count as minus infinity (never
-// chosen while an allowed expert is left, however negative the biased scores are).
+// chosen while an allowed expert is left, however negative the biased scores are); 4 = group score
+// like 2, exclusion like 3.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ logits, int64_t stride, int n_tok,
                                                         int E, int k, int renorm, int scoring,
@@ -92,7 +93,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ lo
           b2 = x;
         }
       }
-      gscore = group_mode == 2 ? b1 + (gs > 1 ? b2 : 0.f) : b1;
+      gscore = group_mode == 2 || group_mode == 4 ? b1 + (gs > 1 ? b2 : 0.f) : b1;
     }
     int chosen = 0;  // bit set on the lanes whose group is selected
     for (int j = 0; j < topk_group; ++j) {
@@ -118,7 +119,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ lo
 #pragma unroll
     for (int i = 0; i < MAXV; ++i) {
       const int e = lane + 64 * i;
-      if (e < E && !s_gsel[wave][e / gs]) key[i] = group_mode == 3 ? OME_NEG_INF : 0.f;
+      if (e < E && !s_gsel[wave][e / gs]) key[i] = group_mode >= 3 ? OME_NEG_INF : 0.f;
     }
   }
   float picked_sum = 0.f;

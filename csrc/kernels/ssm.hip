@@ -7,7 +7,8 @@
 //   ome_ssm_scan         : the selective scan  h <- exp(dt*A) h + dt * B x,  y = C.h + D x
 //                          (dt = softplus(dt + dt_bias) clamped below), recurrent over the rows of
 //                          each sequence, state in fp32 per (slot, head, p, n)
-//   ome_gated_rmsnorm    : out = w * groupRMSNorm(y * silu(z))  (norm_first: w[:group] * groupRMSNorm(y) * silu(z))
+//   ome_gated_rmsnorm    : out = w * groupRMSNorm(y * silu(z))  (norm_first: w[:group] * groupRMSNorm(y) * silu(z),
+//                          or * sigmoid(z))
 //
 // Sequences are described by cu[S+1] (row ranges), slot[S] (state row) and reset[S] (1 = start
 // from zero state: a sequence's first prefill chunk).  Decode is the S = batch, one-row case, so
@@ -188,7 +189,7 @@ __global__ __launch_bounds__(256) void gated_rmsnorm_kernel(const T* __restrict_
                                                             int64_t out_stride, int group, float eps, int mode) {
   __shared__ float red[4];
   const int norm_first = mode & 1;
-  const bool exact = (mode & 2) != 0;
+  const bool exact = (mode & 2) != 0, sig = (mode & 4) != 0;   // sig: sigmoid(z) instead of silu(z) (exact, norm first)
   const int row = blockIdx.y, g0 = blockIdx.x * group;
   const T* yr = y + (int64_t)row * y_stride + g0;
   const T* zr = z + (int64_t)row * z_stride + g0;
@@ -202,7 +203,7 @@ __global__ __launch_bounds__(256) void gated_rmsnorm_kernel(const T* __restrict_
   T* orow = out + (int64_t)row * out_stride + g0;
   for (int i = threadIdx.x; i < group; i += 256) {
     if (exact) {        // one rounding, at the store (models that keep their norms in fp32)
-      const float zs = silu_f((float)zr[i]);
+      const float zs = sig ? 1.f / (1.f + __expf(-(float)zr[i])) : silu_f((float)zr[i]);
       orow[i] = (T)(norm_first ? (float)yr[i] * rs * (float)w[i] * zs : (float)yr[i] * zs * rs * (float)w[g0 + i]);
     } else if (norm_first) {   // Qwen3-Next: w (per group channel) * norm(y), then * silu(z)
       const float t = (float)(T)((float)(T)((float)yr[i] * rs) * (float)w[i]);
@@ -214,6 +215,47 @@ __global__ __launch_bounds__(256) void gated_rmsnorm_kernel(const T* __restrict_
   }
 }
 
+// Small groups in exact mode, norm first: one wave per group, V neighbouring elements per lane and pass.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void gated_rmsnorm_wave_kernel(const T* __restrict__ y, int64_t y_stride,
+                                                                 const T* __restrict__ z, int64_t z_stride,
+                                                                 const T* __restrict__ w, T* __restrict__ out,
+                                                                 int64_t out_stride, int64_t n, int per_row, int group,
+                                                                 float eps, int sig) {
+  typedef T vec __attribute__((ext_vector_type(V)));
+  const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (id >= n) return;
+  const int lane = threadIdx.x & 63, g0 = (int)(id % per_row) * group;
+  const int64_t row = id / per_row;
+  constexpr int NP = 8 / V;   // passes: groups of up to 512
+  vec yv[NP], zv[NP];
+  float ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int i = (lane + 64 * p) * V;
+    if (i < group) {
+      yv[p] = *reinterpret_cast<const vec*>(y + row * y_stride + g0 + i);
+      zv[p] = *reinterpret_cast<const vec*>(z + row * z_stride + g0 + i);
+#pragma unroll
+      for (int e = 0; e < V; ++e) ss += (float)yv[p][e] * (float)yv[p][e];
+    }
+  }
+  const float rs = 1.f / sqrtf(wave_sum(ss) / (float)group + eps);
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int i = (lane + 64 * p) * V;
+    if (i < group) {
+      const vec wv = *reinterpret_cast<const vec*>(w + i);
+      vec o;
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float zz = (float)zv[p][e], gate = 1.f / (1.f + __expf(-zz));
+        o[e] = (T)((float)yv[p][e] * rs * (float)wv[e] * (sig ? gate : zz * gate));
+      }
+      *reinterpret_cast<vec*>(out + row * out_stride + g0 + i) = o;
+    }
+  }
+}
 
 // Any tap count 1 <= K <= 32 (the templated kernels cover 2..6): same arguments, runtime loops.
 template <typename T>
@@ -423,9 +465,30 @@ OME_API int ome_ssm_scan(const void* x, int64_t x_stride, const void* dt, int64_
 
 OME_API int ome_gated_rmsnorm(const void* y, int64_t y_stride, const void* z, int64_t z_stride, const void* w,
                               void* out, int64_t out_stride, int rows, int I, int group, float eps,
-                              int norm_first, int f32, hipStream_t stream) {   // norm_first | 2: no intermediate rounding
+                              int norm_first, int f32, hipStream_t stream) {
+  // norm_first | 2: no intermediate rounding | 4: sigmoid gate (with 1 and 2)
   if (rows <= 0) return 0;
-  if (group <= 0 || I % group != 0) return -2;
+  if (group <= 0 || I % group != 0 || ((norm_first & 4) && (norm_first & 3) != 3)) return -2;
+  if ((norm_first & 3) == 3 && group <= 512 && group % 2 == 0) {
+    const int esz = f32 ? 4 : 2;
+    auto al = [&](const void* p, int64_t stride) { return (((uintptr_t)p | (uintptr_t)(stride * esz)) & (2 * esz - 1)) == 0; };
+    if (al(y, y_stride) && al(z, z_stride) && al(w, 0) && al(out, out_stride)) {
+      const int per_row = I / group, sig = (norm_first & 4) != 0;
+      const int64_t n = (int64_t)rows * per_row;
+      if (n > (int64_t)4 * 0x7fffffff) return -3;
+      const int nblk = (int)((n + 3) / 4);
+      if (f32)
+        gated_rmsnorm_wave_kernel<float, 2><<<nblk, 256, 0, stream>>>((const float*)y, y_stride, (const float*)z, z_stride,
+                                                                      (const float*)w, (float*)out, out_stride, n, per_row,
+                                                                      group, eps, sig);
+      else
+        gated_rmsnorm_wave_kernel<bf16, 2><<<nblk, 256, 0, stream>>>((const bf16*)y, y_stride, (const bf16*)z, z_stride,
+                                                                     (const bf16*)w, (bf16*)out, out_stride, n, per_row, group,
+                                                                     eps, sig);
+      OME_CHECK_LAUNCH();
+      return 0;
+    }
+  }
   dim3 grid(I / group, rows);
   if (f32)
     gated_rmsnorm_kernel<float><<<grid, 256, 0, stream>>>((const float*)y, y_stride, (const float*)z, z_stride,

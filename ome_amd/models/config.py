@@ -169,8 +169,8 @@ def layer_runs(c: dict[str, Any]) -> list[tuple[int, int]]:
 
 
 def _layer_list_keys(c: dict[str, Any]) -> dict[str, Any]:
-    """Layer-list configs (``architecture: Zavilorn`` / ``Metitar`` / ``Milenex`` / ``Nivasun`` / ``Pagatar``): ``layers`` is a
-    list of blocks, each with its mixer ``type``, the mixer's own sizes and its feed-forward.  The
+    """Layer-list configs (``architecture: Zavilorn`` / ``Metitar`` / ``Milenex`` / ``Nivasun`` / ``Pagatar`` /
+    ``Gisirax``): ``layers`` is a list of blocks, each with its mixer ``type``, the mixer's own sizes and its feed-forward.  The
     standard keys describe the envelope the runtime sizes its workspaces by (widest attention layer,
     fewest kv heads); the model reads the per-layer entries from ``extra``.  ``num_hidden_layers``
     counts layer RUNS (a looped span counts once per pass: every pass owns cache pages)."""
@@ -230,9 +230,22 @@ def yarn_rope_table(base: float, rot_dim: int, max_pos: int, scaling: dict | Non
     return cs.to(device) if device is not None else cs
 
 
-def plain_rope_table(base: float, rot_dim: int, max_pos: int, device=None) -> torch.Tensor:
-    """[max_pos, rot_dim] fp32 (cos | sin) for unscaled rotary frequencies base^(-2i/rot_dim)."""
+def band_scaled(inv: torch.Tensor, factor: float, low: float, high: float, original: float) -> torch.Tensor:
+    """Llama-3.1 frequency scaling by wavelength band: with l = 2 pi / f, frequencies of l > original /
+    low are divided by ``factor``, those of l < original / high stay, the ones between are blended
+    linearly in original / l.  fp64 in, fp64 out."""
+    wl = 2 * math.pi / inv
+    smooth = (original / wl - low) / (high - low) if high != low else torch.ones_like(inv)
+    mid = (wl <= original / low) & (wl >= original / high)
+    return torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, torch.where(wl > original / low, inv / factor, inv))
+
+
+def plain_rope_table(base: float, rot_dim: int, max_pos: int, device=None, scaling: dict | None = None) -> torch.Tensor:
+    """[max_pos, rot_dim] fp32 (cos | sin) for rotary frequencies base^(-2i/rot_dim); ``scaling`` =
+    {factor, low, high, original}: :func:`band_scaled` (None: unscaled).  Built in fp64."""
     inv = 1.0 / (float(base) ** (torch.arange(0, rot_dim, 2, dtype=torch.float64) / rot_dim))
+    if scaling:
+        inv = band_scaled(inv, *(float(scaling[k]) for k in ("factor", "low", "high", "original")))
     fr = torch.outer(torch.arange(max_pos, dtype=torch.float64), inv)
     cs = torch.cat([fr.cos(), fr.sin()], -1).float()
     return cs.to(device) if device is not None else cs
@@ -763,15 +776,8 @@ def rope_cos_sin(cfg: ModelConfig, max_pos: int, device=None) -> torch.Tensor:
     if rtype == "linear":
         pos = pos / sc["factor"]
     elif rtype == "llama3":
-        factor = sc["factor"]
-        lf, hf = sc.get("low_freq_factor", 1.0), sc.get("high_freq_factor", 4.0)
-        old = sc.get("original_max_position_embeddings", 8192)
-        low_wl, high_wl = old / lf, old / hf
-        wl = 2 * math.pi / inv
-        smooth = (old / wl - lf) / (hf - lf)
-        scaled = torch.where(wl > low_wl, inv / factor, inv)
-        mid = (wl <= low_wl) & (wl >= high_wl)
-        inv = torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, scaled)
+        inv = band_scaled(inv, sc["factor"], sc.get("low_freq_factor", 1.0), sc.get("high_freq_factor", 4.0),
+                          sc.get("original_max_position_embeddings", 8192))
     elif rtype == "yarn":
         factor = sc["factor"]
         old = sc.get("original_max_position_embeddings", 4096)

@@ -1,11 +1,16 @@
 """Token mixers and feed-forwards as parameterised building blocks (every size and constant is a
 constructor argument), for decoders that assemble their layers from a per-layer list.
 
-* :class:`GatedWindowAttention` -- grouped-query attention over the paged KV cache with a sliding
-  window that keeps the sequence's first tokens visible, projection-wide q / k RMSNorm, partial
-  rotary embedding (interleaved or half-split pairs) and a sigmoid output gate;
+* :class:`GatedWindowAttention` -- grouped-query attention over the paged KV cache with an optional
+  sliding window that keeps the sequence's first tokens visible, optional projection-wide q / k
+  RMSNorm, partial rotary embedding (interleaved or half-split pairs, optionally scaled by
+  wavelength bands), an optional constant sink and an optional sigmoid output gate;
 * :class:`GatedDeltaMixer` -- the gated delta rule (short causal convolutions, unit-norm q / k,
   per-head decay and write strength, fp32 state per request slot);
+* :class:`ChannelDeltaMixer` -- the same with one decay per head and key channel and low-rank
+  decay and output-gate projections;
+* :class:`LightningAttention` -- linear attention with one constant decay per head;
+* :class:`ParallelMixers` -- two of these blocks side by side on one input (one fused projection);
 * :class:`Mamba2Mixer` -- Mamba-2 / SSD selective scan with grouped B / C and a gated group norm;
 * :class:`ClampedGLU` -- gated feed-forward ``min(g, L) * sigmoid(1.702 min(g, L)) * (clamp(u, -L, L) + 1)``;
 * :class:`LatentAttention` -- multi-head latent attention (low-rank queries, one cached latent +
@@ -56,6 +61,13 @@ class MixerCtx:
     kv: PagedKVCache
     seqs: tuple
     cache: dict = field(default_factory=dict)   # tensors derived once per step and shared by the layers
+
+    def seq_rows(self, h: torch.Tensor):
+        """``ops.seq_rows`` of the step for row-parallel kernels of stateful mixers (None on the CPU path)."""
+        rows = self.cache.get("rows")
+        if rows is None and h.is_cuda:
+            rows = self.cache["rows"] = ops.seq_rows(self.seqs, h.shape[0])
+        return rows
 
 
 MAX_HEAD_GROUP = 16   # query heads per kv head one launch of the paged attention kernels takes
@@ -118,46 +130,65 @@ class GatedWindowAttention(_Block):
     """q = W_q h, k = W_k h, v = W_v h; q and k each RMS-normalised over the WHOLE projection
     (all heads at once, weights of that width); rotary on the first ``rot_dims`` dims of every
     head; score = q.k * ``scale``; query i sees key j <= i when i - j < ``window`` or
-    j < ``keep_first``; softmax; heads * sigmoid(W_g h); W_o.  Checkpoint tensors ``q k v q.norm
-    k.norm g o``."""
+    j < ``keep_first``; softmax; heads * sigmoid(W_g h); W_o.  Checkpoint tensors ``q k v [q.norm
+    k.norm] [g] o``.
+
+    Options: ``wide_norm`` False -- q and k are not normed; ``gated`` False -- no output gate;
+    ``rot_scaling`` -- wavelength-band scaling of the rotary frequencies (``config.band_scaled``);
+    ``sink`` -- a constant score that joins every head's softmax denominator (no key, no value;
+    0.0: one is added to the denominator).  ``forward(h, ctx, p)``: the input projection was made
+    by the caller (``ParallelMixers``)."""
 
     def __init__(self, layer: int, width: int, heads: int, kv_heads: int, dim: int, vdim: int, window: int,
                  keep_first: int, rot_base: float, rot_dims: int, scale: float, eps: float, max_positions: int,
-                 device, dtype, interleaved: bool = True):
+                 device, dtype, interleaved: bool = True, wide_norm: bool = True, gated: bool = True,
+                 rot_scaling: dict | None = None, sink: float | None = None):
         super().__init__(device, dtype)
-        if heads % kv_heads or heads // kv_heads > 16:
-            raise ValueError(f"attention: {heads} query heads over {kv_heads} kv heads (groups of <= 16 supported)")
+        if heads % kv_heads:
+            raise ValueError(f"attention: {heads} query heads do not divide over {kv_heads} kv heads")
         self.layer, self.width, self.Hq, self.Hkv, self.dim, self.vdim = layer, width, heads, kv_heads, dim, vdim
         self.window, self.keep_first = int(window) if window and window > 0 else -1, int(keep_first)
         self.rot_dims, self.scale, self.eps, self.interleaved = int(rot_dims), float(scale), float(eps), interleaved
+        self.wide_norm, self.gated = bool(wide_norm), bool(gated)
         self.D = attn_tile_dim(max(dim, vdim))
-        self.cos_sin = plain_rope_table(rot_base, self.rot_dims, max_positions, self.device) if rot_dims else \
+        self.cos_sin = plain_rope_table(rot_base, self.rot_dims, max_positions, self.device, rot_scaling) if rot_dims else \
             torch.zeros(max_positions, 0, device=self.device)
         self.nq, self.nk, self.nv = heads * dim, kv_heads * dim, kv_heads * vdim
+        self.rows = self.nq + self.nk + self.nv + (heads * vdim if gated else 0)     # of the input projection
         self.w_in = self.qn = self.kn = self.w_o = None
+        self.sink = None if sink is None else torch.full((heads,), float(sink), dtype=torch.float32, device=self.device)
 
     def load(self, t: dict) -> None:
-        self.w_in = self._put(torch.cat([t["q"], t["k"], t["v"], t["g"]], 0))
-        self.qn, self.kn = self._put(t["q.norm"]), self._put(t["k.norm"])
+        self.w_in = self._put(torch.cat([t["q"], t["k"], t["v"]] + ([t["g"]] if self.gated else []), 0))
+        if tuple(self.w_in.shape) != (self.rows, self.width):
+            raise ValueError(f"attention: projections {tuple(self.w_in.shape)} != [{self.rows}, {self.width}]")
+        if self.wide_norm:
+            self.qn, self.kn = self._put(t["q.norm"]), self._put(t["k.norm"])
         self.w_o = self._put(t["o"])
 
     def init_random(self, gen, std: float) -> None:
-        self.w_in = self._rand(gen, self.nq + self.nk + self.nv + self.Hq * self.vdim, self.width, std=std)
-        self.qn = torch.ones(self.nq, dtype=self.dtype, device=self.device)
-        self.kn = torch.ones(self.nk, dtype=self.dtype, device=self.device)
+        self.w_in = self._rand(gen, self.rows, self.width, std=std)
+        if self.wide_norm:
+            self.qn = torch.ones(self.nq, dtype=self.dtype, device=self.device)
+            self.kn = torch.ones(self.nk, dtype=self.dtype, device=self.device)
         self.w_o = self._rand(gen, self.width, self.Hq * self.vdim, std=std)
 
-    def forward(self, h: torch.Tensor, ctx: MixerCtx) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, ctx: MixerCtx, p: torch.Tensor | None = None) -> torch.Tensor:
         T = h.shape[0]
         nq, nk, nv = self.nq, self.nk, self.nv
-        p = linear(h, self.w_in)                                   # [T, q | k | v | gate]
+        if p is None:
+            p = linear(h, self.w_in)                               # [T, q | k | v (| gate)]
         q = torch.empty(T, self.Hq, self.D, dtype=h.dtype, device=h.device)
         k_cache, v_cache = ctx.kv.layer(self.layer)
         ops.wide_norm_rope_cache(p[:, :nq], p[:, nq:nq + nk], p[:, nq + nk:nq + nk + nv], ctx.meta.positions,
                                  self.cos_sin, self.rot_dims, self.interleaved, self.qn, self.kn, self.eps, q,
                                  k_cache, v_cache, ctx.meta.slots, self.Hq, self.Hkv, self.dim, self.vdim)
-        a = paged_attention(q, k_cache, v_cache, ctx.meta, self.scale, self.window, self.keep_first)
-        return linear(ops.head_gate(a, p[:, nq + nk + nv:], self.vdim, 0), self.w_o)
+        a = paged_attention(q, k_cache, v_cache, ctx.meta, self.scale, self.window, self.keep_first, self.sink)
+        if self.gated:
+            return linear(ops.head_gate(a, p[:, nq + nk + nv:], self.vdim, 0), self.w_o)
+        if self.D != self.vdim:
+            a = a[:, :, :self.vdim].reshape(T, self.Hq * self.vdim)
+        return linear(a.view(T, self.Hq * self.vdim), self.w_o)
 
 
 class GatedDeltaMixer(_Block):
@@ -208,6 +239,176 @@ class GatedDeltaMixer(_Block):
                          self.A_log, self.dt_bias, self.rec_state, cu, slot, reset, Hv, self.Hk)
         o = ops.gated_rmsnorm(o, p[:, cd:cd + vd], self.gnorm, self.dv, self.eps, norm_first=True, exact=True)
         return linear(o, self.w_o)
+
+
+class ChannelDeltaMixer(_Block):
+    """Gated delta rule with one decay per head and key channel.  q, k (``kv_heads`` x ``dim``) and v
+    (``heads`` x ``vdim``) pass a causal depthwise convolution of ``conv`` taps + SiLU; q, k become unit
+    vectors per head (q also times dim^-1/2); with g = exp(-exp(A_log_h) softplus(W_a2 W_a1 h +
+    dt_bias)) (``heads`` x ``dim``) and beta = sigmoid(W_b h):
+    S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q.
+    Output: each head's o over its root mean square, times a weight shared by the heads, times
+    sigmoid(W_g2 W_g1 h); W_o.  Checkpoint tensors ``q q.conv k k.conv v v.conv b A_log a1 a2
+    dt_bias g1 g2 norm o`` (the ranks are the rows of a1 and g1); state: conv tail [slots, C, conv -
+    1], S^T [slots, heads, vdim, dim] fp32.
+
+    Two GEMMs in front of one op (``ops.channel_delta``): the fused input projection [q | k | v |
+    a1 | g1 | b] and the low-rank second factors as ONE block-diagonal product over its a1 | g1
+    columns (the parts start on multiples of 8 columns, padded with zero rows)."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, conv: int, eps: float, device,
+                 dtype):
+        super().__init__(device, dtype)
+        if heads % kv_heads:
+            raise ValueError(f"gated delta rule: {heads} value heads over {kv_heads} key heads")
+        if dim > ops.STATE_DIM_MAX or not 1 <= conv <= 32:
+            raise ValueError(f"gated delta rule: key width {dim} (at most {ops.STATE_DIM_MAX}) or {conv} taps (1 to 32)")
+        self.width, self.Hv, self.Hk, self.dk, self.dv, self.K, self.eps = width, heads, kv_heads, dim, vdim, conv, float(eps)
+        self.kd, self.vd = kv_heads * dim, heads * vdim
+        self.cd = 2 * self.kd + self.vd
+        self.w_in = self.conv_w = self.A_log = self.dt_bias = self.w_lr = self.gnorm = self.w_o = None
+        self.conv_state = self.rec_state = None
+        self.lr0 = self.lrw = self.b0 = 0                     # where the low-rank part starts / its width / the write strengths
+
+    def _fuse(self, qkv: torch.Tensor, a1: torch.Tensor, g1: torch.Tensor, b: torch.Tensor, a2: torch.Tensor,
+              g2: torch.Tensor) -> None:
+        ra, rg = a1.shape[0], g1.shape[0]
+        up8 = lambda n: -(-n // 8) * 8   # noqa: E731
+        self.lr0, self.lrw = up8(self.cd), up8(ra + rg)
+        self.b0 = self.lr0 + self.lrw
+        w = qkv.new_zeros(up8(self.b0 + self.Hv), self.width)
+        w[:self.cd] = qkv
+        w[self.lr0:self.lr0 + ra + rg] = torch.cat([a1, g1], 0)
+        w[self.b0:self.b0 + self.Hv] = b
+        na = self.Hv * self.dk
+        w2 = qkv.new_zeros(na + self.vd, self.lrw)
+        w2[:na, :ra], w2[na:, ra:ra + rg] = a2, g2
+        self.w_in, self.w_lr = self._put(w), self._put(w2)
+
+    def load(self, t: dict) -> None:
+        W, H = self.width, self.Hv
+        want = {"q": (self.kd, W), "k": (self.kd, W), "v": (self.vd, W), "b": (H, W), "a2": (H * self.dk, t["a1"].shape[0]),
+                "g2": (self.vd, t["g1"].shape[0]), "o": (W, self.vd), "q.conv": (self.kd, self.K), "k.conv": (self.kd, self.K),
+                "v.conv": (self.vd, self.K), "A_log": (H,), "dt_bias": (H * self.dk,), "norm": (self.dv,)}
+        for n, shape in want.items():
+            if tuple(t[n].shape) != shape:
+                raise ValueError(f"gated delta rule: {n} {tuple(t[n].shape)} != {list(shape)}")
+        self._fuse(torch.cat([t["q"], t["k"], t["v"]], 0), t["a1"], t["g1"], t["b"], t["a2"], t["g2"])
+        self.conv_w = self._put(torch.cat([t["q.conv"], t["k.conv"], t["v.conv"]], 0))
+        self.A_log, self.dt_bias = self._put(t["A_log"], torch.float32), self._put(t["dt_bias"], torch.float32)
+        self.gnorm, self.w_o = self._put(t["norm"]), self._put(t["o"])
+
+    def init_random(self, gen, std: float) -> None:
+        f32 = dict(dtype=torch.float32, device=self.device)
+        r, W = self.dv, self.width                            # (ranks as wide as a value head)
+        self._fuse(self._rand(gen, self.cd, W, std=std), self._rand(gen, r, W, std=std), self._rand(gen, r, W, std=std),
+                   self._rand(gen, self.Hv, W, std=std), self._rand(gen, self.Hv * self.dk, r, std=std),
+                   self._rand(gen, self.vd, r, std=std))
+        self.conv_w = self._rand(gen, self.cd, self.K, std=0.3)
+        self.A_log = torch.log(torch.linspace(0.02, 0.5, self.Hv, **f32))
+        self.dt_bias = torch.linspace(-1.0, 1.0, self.Hv * self.dk, **f32)
+        self.gnorm = torch.ones(self.dv, dtype=self.dtype, device=self.device)
+        self.w_o = self._rand(gen, W, self.vd, std=std)
+
+    def alloc_state(self, slots: int) -> None:
+        self.conv_state = torch.zeros(slots, self.cd, self.K - 1, dtype=self.dtype, device=self.device)
+        self.rec_state = torch.zeros(slots, self.Hv, self.dv, self.dk, dtype=torch.float32, device=self.device)
+
+    def forward(self, h: torch.Tensor, ctx: MixerCtx) -> torch.Tensor:
+        p = linear(h, self.w_in)                                  # [T, q | k | v | a1 | g1 | b]
+        z = linear(p[:, self.lr0:self.lr0 + self.lrw], self.w_lr)  # [T, decay | output gate]
+        single = ctx.meta.is_decode
+        rows = None if single else ctx.seq_rows(h)
+        o = ops.channel_delta(p[:, :self.cd], self.conv_w, self.conv_state, z, p[:, self.b0:self.b0 + self.Hv], self.A_log,
+                              self.dt_bias, self.gnorm, self.eps, self.rec_state, ctx.seqs, self.Hk, rows=rows,
+                              single_rows=single)
+        return linear(o, self.w_o)
+
+
+class LightningAttention(_Block):
+    """Linear attention with a constant decay per head: q = silu(W_q h), k = silu(W_k h), v = silu(W_v
+    h) (``heads`` x ``dim`` / ``vdim``); S <- decay_h S + k v^T, o = S^T q; the concatenated heads
+    are RMS-normed together with a weight, times sigmoid(W_g h); W_o.  Checkpoint tensors ``q k v g
+    norm o``; state S^T [slots, heads, vdim, dim] fp32.  ``forward(h, ctx, p)``: the input
+    projection was made by the caller."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay, eps: float, device, dtype):
+        super().__init__(device, dtype)
+        if len(decay) != heads:
+            raise ValueError(f"lightning attention: {len(decay)} decays for {heads} heads")
+        if dim > ops.STATE_DIM_MAX:
+            raise ValueError(f"lightning attention: key width {dim} exceeds {ops.STATE_DIM_MAX}")
+        self.width, self.H, self.dim, self.vdim, self.eps = width, heads, dim, vdim, float(eps)
+        self.decay = torch.tensor([float(d) for d in decay], dtype=torch.float32, device=self.device)
+        self.nk, self.nv = heads * dim, heads * vdim
+        self.rows = 2 * (self.nk + self.nv)                       # of the input projection
+        self.w_in = self.gnorm = self.w_o = None
+        self.rec_state = None
+
+    def load(self, t: dict) -> None:
+        self.w_in = self._put(torch.cat([t["q"], t["k"], t["v"], t["g"]], 0))
+        if tuple(self.w_in.shape) != (self.rows, self.width):
+            raise ValueError(f"lightning attention: projections {tuple(self.w_in.shape)} != [{self.rows}, {self.width}]")
+        self.gnorm, self.w_o = self._put(t["norm"]), self._put(t["o"])
+
+    def init_random(self, gen, std: float) -> None:
+        self.w_in = self._rand(gen, self.rows, self.width, std=std)
+        self.gnorm = torch.ones(self.nv, dtype=self.dtype, device=self.device)
+        self.w_o = self._rand(gen, self.width, self.nv, std=std)
+
+    def alloc_state(self, slots: int) -> None:
+        self.rec_state = torch.zeros(slots, self.H, self.vdim, self.dim, dtype=torch.float32, device=self.device)
+
+    def forward(self, h: torch.Tensor, ctx: MixerCtx, p: torch.Tensor | None = None) -> torch.Tensor:
+        if p is None:
+            p = linear(h, self.w_in)                              # [T, q | k | v | gate]
+        n = self.nk
+        o = ops.lightning_scan(p[:, :n], p[:, n:2 * n], p[:, 2 * n:2 * n + self.nv], self.decay, self.rec_state, ctx.seqs,
+                               single_rows=ctx.meta.is_decode)
+        o = ops.gated_rmsnorm(o, p[:, 2 * n + self.nv:], self.gnorm, self.nv, self.eps, norm_first=True, exact=True,
+                              gate="sigmoid")
+        return linear(o, self.w_o)
+
+
+class ParallelMixers(_Block):
+    """Two mixers side by side on one input: their input projections run as ONE GEMM, the right one's
+    columns starting on a multiple of 8.  ``forward`` returns the two outputs (how they are joined
+    is the caller's matter).  Both blocks have ``rows`` (of their projection), ``w_in`` and
+    ``forward(h, ctx, p)``."""
+
+    def __init__(self, left, right, device, dtype):
+        super().__init__(device, dtype)
+        self.left, self.right = left, right
+        self.r0 = -(-left.rows // 8) * 8                          # the right block's first column
+        self.w_in = None
+
+    def _fuse(self) -> None:
+        w = self.left.w_in.new_zeros(-(-(self.r0 + self.right.rows) // 8) * 8, self.left.width)
+        w[:self.left.rows], w[self.r0:self.r0 + self.right.rows] = self.left.w_in, self.right.w_in
+        self.w_in = w
+        self.left.w_in = self.right.w_in = None
+
+    def load(self, left: dict, right: dict) -> None:
+        self.left.load(left)
+        self.right.load(right)
+        self._fuse()
+
+    def init_random(self, gen, std: float) -> None:
+        self.left.init_random(gen, std)
+        self.right.init_random(gen, std)
+        self._fuse()
+
+    def alloc_state(self, slots: int) -> None:
+        self.left.alloc_state(slots)
+        self.right.alloc_state(slots)
+
+    def tensors(self) -> list[torch.Tensor]:
+        return super().tensors() + self.left.tensors() + self.right.tensors()
+
+    def forward(self, h: torch.Tensor, ctx: MixerCtx) -> tuple[torch.Tensor, torch.Tensor]:
+        p = linear(h, self.w_in)
+        return (self.left.forward(h, ctx, p[:, :self.left.rows]),
+                self.right.forward(h, ctx, p[:, self.r0:self.r0 + self.right.rows]))
 
 
 class Mamba2Mixer(_Block):
@@ -690,9 +891,7 @@ class ConvRotaryAttention(_Block):
         p = linear(h, self.w_in)                                   # [T, q | k | v (| gate)]
         q = torch.empty(T, self.Hq, self.D, dtype=h.dtype, device=h.device)
         k_cache, v_cache = ctx.kv.layer(self.layer)
-        rows = ctx.cache.get("rows")
-        if rows is None and h.is_cuda:
-            rows = ctx.cache["rows"] = ops.seq_rows(ctx.seqs, T)
+        rows = ctx.seq_rows(h)
         v_out = None
         if self.v_mix == "first":
             v_out = ctx.cache["v_first"] = torch.empty(T, nv, dtype=h.dtype, device=h.device)
@@ -841,7 +1040,9 @@ class GroupRoutedMoE(_Block):
     ``scoring``: "softmax", or "sigmoid" = every score on its own, s = sigmoid(W_r h);
     ``renorm``: the chosen scores are divided by their sum (= a softmax over the chosen logits
     alone); ``router_bias``: the router has a bias ``router.b`` that is part of the logits;
-    ``correction`` False: no choice-only correction tensor.
+    ``correction`` False: no choice-only correction tensor; ``group_score``: a group scores by its
+    best choice score ("max") or by the sum of its two best ("top2"); ``routed_scale``: a factor on
+    the weights.
     Checkpoint tensors ``router [router.b] [correction] e<j>.gate|up|down [shared.gate|up|down|sg]``.
 
     The router and the shared gate are one fp32-result GEMM (``[W_r; w_sg]``).  Experts run on the
@@ -851,9 +1052,11 @@ class GroupRoutedMoE(_Block):
 
     def __init__(self, width: int, experts: int, top: int, ff: int, limit: float, groups: int, keep: int,
                  shared_ff: int, shared_limit: float, device, dtype, act: int = 2, renorm: bool = False,
-                 router_bias: bool = False, correction: bool = True, scoring: str = "softmax"):
+                 router_bias: bool = False, correction: bool = True, scoring: str = "softmax", group_score: str = "max",
+                 routed_scale: float = 1.0):
         super().__init__(device, dtype)
-        self.scoring = scoring
+        self.scoring, self.routed_scale = scoring, float(routed_scale)
+        self.group_mode = 0 if groups == 1 else {"max": 3, "top2": 4}[group_score]
         if groups < 1 or experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups):
             raise ValueError(f"moe: {experts} experts in {groups} groups, {keep} kept, top {top}")
         if experts > 512 or top > 16:
@@ -894,7 +1097,7 @@ class GroupRoutedMoE(_Block):
         T, W = h.shape
         logits = ops.lm_head_f32(h, self.w_router)                        # fp32 [T, E (+ shared gate)]
         tw, tid = ops.moe_route(logits[:, :self.E], self.k, self.renorm, self.scoring, bias=self.correction,
-                                n_group=self.groups, topk_group=self.keep, group_mode=3 if self.groups > 1 else 0,
+                                n_group=self.groups, topk_group=self.keep, group_mode=self.group_mode,
                                 logit_bias=self.router_b)
         sh = None
         if self.sff:
@@ -902,9 +1105,9 @@ class GroupRoutedMoE(_Block):
                                 row_gate=logits[:, self.E])
             sh = linear(a, self.w_sd)
         if self.grouped_ok(h):
-            return ops.fused_moe(h, tw, tid, self.w13, self.w2, act=self.act, limit=self.limit,
+            return ops.fused_moe(h, tw, tid, self.w13, self.w2, act=self.act, limit=self.limit, scale=self.routed_scale,
                                  add=sh.contiguous() if sh is not None else None)
-        wd = torch.zeros(T, self.E, dtype=torch.float32, device=h.device).scatter_(1, tid.long(), tw)
+        wd = torch.zeros(T, self.E, dtype=torch.float32, device=h.device).scatter_(1, tid.long(), tw * self.routed_scale)
         gu = torch.matmul(h, self.w13)                                    # [E, T, 2 ff]
         hh = ops.act_and_mul(gu.view(self.E * T, 2 * self.ff), self.act, limit=self.limit).view(self.E, T, self.ff)
         y = (torch.bmm(hh, self.w2).float() * wd.t()[:, :, None]).sum(0)

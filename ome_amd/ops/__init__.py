@@ -204,17 +204,20 @@ def gdn_scan(q, k, v, a, b, A_log, dt_bias, state, cu, slot, reset, Hv: int, Hk:
 
 
 def gated_rmsnorm(y: torch.Tensor, z: torch.Tensor, w: torch.Tensor, group: int, eps: float,
-                  norm_first: bool = False, exact: bool = False) -> torch.Tensor:
+                  norm_first: bool = False, exact: bool = False, gate: str = "silu") -> torch.Tensor:
     """w * groupRMSNorm(y * silu(z)) (Mamba-2 output norm, groups of ``group`` channels);
     ``norm_first``: w[:group] * groupRMSNorm(y) * silu(z) (Qwen3-Next, ``w`` shared by the groups).
     ``exact``: the whole expression in fp32 with one rounding at the store (default: the
-    normalised value is rounded to the model dtype before the scale, as HF's modules do)."""
+    normalised value is rounded to the model dtype before the scale, as HF's modules do).
+    ``gate="sigmoid"``: sigmoid(z) in place of silu(z) (with ``norm_first`` and ``exact``)."""
+    assert gate == "silu" or (gate == "sigmoid" and norm_first and exact)
     if not _gpu(y):
-        return ref.gated_rmsnorm(y, z, w, group, eps, norm_first, exact)
+        return ref.gated_rmsnorm(y, z, w, group, eps, norm_first, exact, gate)
     T, I = y.shape
     out = torch.empty(T, I, dtype=y.dtype, device=y.device)
     call("ome_gated_rmsnorm", y.data_ptr(), y.stride(0), z.data_ptr(), z.stride(0), w.data_ptr(), out.data_ptr(),
-         out.stride(0), T, I, group, float(eps), int(norm_first) | (2 if exact else 0), _f32(y, z, w), stream_ptr())
+         out.stride(0), T, I, group, float(eps), int(norm_first) | (2 if exact else 0) | (4 if gate == "sigmoid" else 0),
+         _f32(y, z, w), stream_ptr())
     return out
 
 
@@ -641,7 +644,8 @@ def moe_route(logits: torch.Tensor, k: int, renorm: bool = True, scoring: str = 
     which only steers the choice).  ``group_mode`` 1/2 =
     DeepSeek-V2 group_limited_greedy / DeepSeek-V3 noaux_tc (with ``bias``); 3 = a group scores by
     its best biased expert and the experts of unchosen groups are excluded outright (minus
-    infinity where modes 1 / 2 set them to 0, which a negative biased score would lose against)."""
+    infinity where modes 1 / 2 set them to 0, which a negative biased score would lose against); 4 =
+    mode 2's group score with mode 3's exclusion."""
     if not _gpu(logits):
         w, ids = ref.moe_route(logits, k, renorm, scoring, bias, n_group, topk_group, group_mode, logit_bias)
         if out_w is not None:
@@ -2102,6 +2106,102 @@ def stream_step(y: torch.Tensor, w: torch.Tensor, groups: int, eps: float, res: 
          _i32(ids).data_ptr(), y.shape[0], ptr(res), res.stride(0) if res is not None else 0, w.data_ptr(), int(groups),
          float(eps), ptr(hist), T * H, int(k), ptr(coef), ptr(x_out), x_out.stride(0) if x_out is not None else 0,
          ptr(out), H, T, H, f32, stream_ptr())
+    return out
+
+
+def tanh_stream(x: torch.Tensor, pre: tuple, out_dtype, post: tuple | None = None, mult: float = 1.0,
+                y: torch.Tensor | None = None, y2: torch.Tensor | None = None, join: tuple | None = None) -> torch.Tensor:
+    """Step of an fp32 residual stream with tanh norms ``D(v) = tanh(alpha v) w + b``, each given as
+    ``(alpha, w, b)``: ``x += mult * D_post(y)`` in place (no ``y``: x stays), returns ``D_pre(x)``
+    rounded to ``out_dtype``.  ``y2``: y is joined from two outputs first, ``(y / rms(y) * w1 + y2 /
+    rms(y2) * w2) / 2`` with ``join`` = (w1, w2, eps); sums, norms and curves are fp32."""
+    if not _gpu(x):
+        return ref.tanh_stream(x, pre, out_dtype, post, mult, y, y2, join)
+    T, H = x.shape
+    pa, pw, pb = post or (0.0, None, None)
+    w1, w2, eps = join or (None, None, 0.0)
+    f32 = _f32(pre[1], pre[2], y, y2, pw, pb, w1, w2)
+    assert x.dtype == torch.float32 and x.stride(1) == 1 and out_dtype == pre[1].dtype
+    for t in (y, y2):
+        assert t is None or (t.shape == x.shape and t.stride(1) == 1)
+    for t in (pre[1], pre[2], pw, pb, w1, w2):
+        assert t is None or (t.numel() == H and t.is_contiguous())
+    out = torch.empty(T, H, dtype=out_dtype, device=x.device)
+    call("ome_tanh_stream", x.data_ptr(), x.stride(0), ptr(y), y.stride(0) if y is not None else 0, ptr(y2),
+         y2.stride(0) if y2 is not None else 0, ptr(w1), ptr(w2), float(eps), float(mult), float(pa), ptr(pw), ptr(pb),
+         float(pre[0]), pre[1].data_ptr(), pre[2].data_ptr(), out.data_ptr(), H, T, H, f32, stream_ptr())
+    return out
+
+
+STATE_DIM_MAX = 512   # key channels per head of the matrix-state recurrences below
+
+
+def channel_delta(qkv: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor, z: torch.Tensor, b: torch.Tensor,
+                  A_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor, eps: float, state: torch.Tensor,
+                  seqs: tuple, Hk: int, rows: tuple | None = None, single_rows: bool = False) -> torch.Tensor:
+    """Core of a gated delta rule with one decay per head and key channel.  ``qkv`` rows [q (Hk*dk) | k
+    (Hk*dk) | v (H*dv)] pass a causal depthwise convolution (``conv_w`` [C, K], tails ``conv_state``
+    [slots, C, K-1]) + SiLU, q and k become unit vectors per head (q also / sqrt(dk)); ``z`` rows hold
+    the decay inputs [H*dk] and the output gate [H*dv]: g = exp(-exp(A_log_h) softplus(z + dt_bias));
+    beta = sigmoid(``b`` [T, H]); per head S <- diag(g) S, u = beta (v - S^T k), S <- S + k u^T, o =
+    S^T q (value head h reads key head h // (H / Hk)); returns o / rms(o) * ``norm_w`` * sigmoid(gate)
+    as [T, H*dv].  ``state`` fp32 [slots, H, dv, dk] (S transposed).  ``seqs`` = (cu, slot, reset);
+    ``rows`` = :func:`seq_rows`; ``single_rows``: every sequence has one row (one launch)."""
+    cu, slot, reset = seqs
+    H, dv, dk = state.shape[1:]
+    T = qkv.shape[0]
+    C, K = conv_w.shape
+    out = torch.empty(T, H * dv, dtype=qkv.dtype, device=qkv.device)
+    assert C == 2 * Hk * dk + H * dv == qkv.shape[1] and z.shape[1] == H * (dk + dv) and b.shape[1] == H and H % Hk == 0
+    if not _gpu(qkv):
+        return ref.channel_delta(qkv, conv_w, conv_state, z, b, A_log, dt_bias, norm_w, eps, state, cu, slot, reset, Hk, out)
+    f32 = _f32(qkv, conv_w, conv_state, z, b, norm_w)
+    assert dk <= STATE_DIM_MAX and qkv.stride(1) == z.stride(1) == b.stride(1) == 1 and norm_w.numel() == dv
+    assert conv_w.is_contiguous() and conv_state.is_contiguous() and tuple(conv_state.shape[1:]) == (C, K - 1)
+    assert state.dtype == torch.float32 and state.is_contiguous()
+    assert A_log.dtype == dt_bias.dtype == torch.float32 and A_log.numel() == H and dt_bias.numel() == H * dk
+    assert A_log.is_contiguous() and dt_bias.is_contiguous() and norm_w.is_contiguous()
+    sp = (_i32(cu).data_ptr(), _i32(slot).data_ptr(), _i32(reset).data_ptr(), slot.shape[0])
+    if single_rows:
+        assert slot.shape[0] == T
+        call("ome_delta_step", qkv.data_ptr(), qkv.stride(0), conv_w.data_ptr(), conv_state.data_ptr(), K, z.data_ptr(),
+             z.stride(0), b.data_ptr(), b.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), norm_w.data_ptr(), float(eps),
+             state.data_ptr(), out.data_ptr(), *sp, H, Hk, dk, dv, f32, stream_ptr())
+        return out
+    first, rslot = rows if rows is not None else seq_rows(seqs, T)
+    dkp = max(16, 1 << (dk - 1).bit_length())
+    ws = torch.empty(T * Hk * (2 * dkp + 1), dtype=torch.float32, device=qkv.device)
+    qn, kn, qk = ws[:T * Hk * dkp], ws[T * Hk * dkp:2 * T * Hk * dkp], ws[2 * T * Hk * dkp:]
+    v = torch.empty(T, H * dv, dtype=qkv.dtype, device=qkv.device)
+    call("ome_delta_prep", qkv.data_ptr(), qkv.stride(0), conv_w.data_ptr(), conv_state.data_ptr(), K, _i32(first).data_ptr(),
+         _i32(rslot).data_ptr(), qn.data_ptr(), kn.data_ptr(), qk.data_ptr(), v.data_ptr(), T, H, Hk, dk, dv, f32, stream_ptr())
+    call("ome_delta_scan", qn.data_ptr(), kn.data_ptr(), qk.data_ptr(), v.data_ptr(), z.data_ptr(), z.stride(0), b.data_ptr(),
+         b.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(), out.data_ptr(), *sp, H, Hk, dk, dv, f32,
+         stream_ptr())
+    if K > 1:
+        call("ome_conv_tail", qkv.data_ptr(), qkv.stride(0), conv_state.data_ptr(), *sp, C, K, f32, stream_ptr())
+    return gated_rmsnorm(out, z[:, H * dk:], norm_w, dv, eps, norm_first=True, exact=True, gate="sigmoid")
+
+
+def lightning_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+                   seqs: tuple, single_rows: bool = False) -> torch.Tensor:
+    """Linear attention with a constant decay per head: S <- decay_h S + silu(k) silu(v)^T, o = S^T
+    silu(q) -> [T, H*dv].  q / k [T, H*dk], v [T, H*dv]: views of one projection (same row stride);
+    ``decay`` fp32 [H]; ``state`` fp32 [slots, H, dv, dk] (S transposed); ``seqs`` = (cu, slot, reset);
+    ``single_rows``: every sequence has one row."""
+    cu, slot, reset = seqs
+    H, dv, dk = state.shape[1:]
+    T = q.shape[0]
+    out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
+    if not _gpu(q):
+        return ref.lightning_scan(q, k, v, decay, state, cu, slot, reset, out)
+    assert q.stride(0) == k.stride(0) == v.stride(0) and q.stride(1) == k.stride(1) == v.stride(1) == 1
+    assert q.shape[1] == k.shape[1] == H * dk and v.shape[1] == H * dv and dk <= STATE_DIM_MAX
+    assert state.dtype == decay.dtype == torch.float32 and state.is_contiguous() and decay.numel() == H and decay.is_contiguous()
+    sp = (_i32(cu).data_ptr(), _i32(slot).data_ptr(), _i32(reset).data_ptr(), slot.shape[0])
+    assert not single_rows or slot.shape[0] == T
+    call("ome_lightning_step" if single_rows else "ome_lightning_scan", q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0),
+         decay.data_ptr(), state.data_ptr(), out.data_ptr(), *sp, H, dk, dv, _f32(q, k, v), stream_ptr())
     return out
 
 

@@ -154,8 +154,12 @@ def gdn_scan(q, k, v, a, b, A_log, dt_bias, state, cu, slot, reset, Hv, Hk, out)
     return out
 
 
-def gated_rmsnorm(y, z, w, group, eps, norm_first=False, exact=False):
+def gated_rmsnorm(y, z, w, group, eps, norm_first=False, exact=False, gate="silu"):
     T, I = y.shape
+    if gate == "sigmoid":   # (norm_first, exact)
+        g = y.float().view(T, I // group, group)
+        g = g * torch.rsqrt(g.pow(2).mean(-1, keepdim=True) + eps) * w.float()[:group]
+        return (g.view(T, I) * torch.sigmoid(z.float())).to(y.dtype)
     if exact:   # fp32 throughout, one rounding at the end
         zs = torch.nn.functional.silu(z.float())
         v = y.float() if norm_first else y.float() * zs
@@ -551,17 +555,18 @@ def moe_route(logits, k: int, renorm: bool, scoring: str = "softmax", bias=None,
               topk_group: int = 1, group_mode: int = 0, logit_bias=None):
     """HF semantics (Mixtral/Qwen softmax top-k; DeepSeek-V2 group_limited_greedy = mode 1,
     DeepSeek-V3 noaux_tc = mode 2 with e_score_correction_bias; mode 3 = the group's best
-    biased score, experts of the other groups excluded outright: minus infinity instead of 0)."""
+    biased score, experts of the other groups excluded outright: minus infinity instead of 0; mode
+    4 = mode 2's group score with mode 3's exclusion)."""
     lf = logits.float() if logit_bias is None else logits.float() + logit_bias.float()
     p = torch.softmax(lf, -1) if scoring == "softmax" else torch.sigmoid(lf)
     key = p + bias.float() if bias is not None else p.clone()
     if group_mode and n_group > 1:
         T, E = key.shape
         grp = key.view(T, n_group, E // n_group)
-        gs = grp.topk(min(2, E // n_group), -1).values.sum(-1) if group_mode == 2 else grp.max(-1).values
+        gs = grp.topk(min(2, E // n_group), -1).values.sum(-1) if group_mode in (2, 4) else grp.max(-1).values
         gidx = gs.topk(topk_group, -1).indices
         gmask = torch.zeros_like(gs, dtype=torch.bool).scatter_(1, gidx, True)
-        key = key.masked_fill(~gmask.repeat_interleave(E // n_group, 1), float("-inf") if group_mode == 3 else 0.0)
+        key = key.masked_fill(~gmask.repeat_interleave(E // n_group, 1), float("-inf") if group_mode >= 3 else 0.0)
     _, ids = torch.topk(key, k, dim=-1)  # ties: torch.topk order is implementation-defined
     w = p.gather(1, ids)
     if renorm:
@@ -937,6 +942,67 @@ def talking_attn(q, k_cache, v_cache, block_tables, row_seq, row_pos, scale, win
         if gate is not None:
             o = o * torch.sigmoid(gate[t].float())[:, None]
         out[t] = o.reshape(-1).to(out.dtype)
+    return out
+
+
+def tanh_stream(x, pre, out_dtype, post=None, mult=1.0, y=None, y2=None, join=None):
+    if y is not None:
+        v = y.float()
+        if y2 is not None:
+            w1, w2, eps = join
+            v = 0.5 * (v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w1.float() +
+                       y2.float() * torch.rsqrt(y2.float().pow(2).mean(-1, keepdim=True) + eps) * w2.float())
+        x += mult * (torch.tanh(post[0] * v) * post[1].float() + post[2].float())
+    return (torch.tanh(pre[0] * x) * pre[1].float() + pre[2].float()).to(out_dtype)
+
+
+def channel_delta(qkv, conv_w, conv_state, z, b, A_log, dt_bias, norm_w, eps, state, cu, slot, reset, Hk, out):
+    Hv, dv, dk = state.shape[1:]
+    kd, na, rep = Hk * dk, Hv * dk, Hv // Hk
+    c = torch.empty(qkv.shape, dtype=torch.float32, device=qkv.device)
+    ssm_conv1d(qkv, conv_w, None, conv_state, cu, slot, reset, c)
+    T = qkv.shape[0]
+
+    def unit(x):
+        x = x.reshape(T, Hk, dk)
+        return (x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + 1e-6)).repeat_interleave(rep, 1)
+
+    q, k, v = unit(c[:, :kd]) * dk ** -0.5, unit(c[:, kd:2 * kd]), c[:, 2 * kd:].reshape(T, Hv, dv)
+    g = torch.exp(-torch.exp(A_log)[:, None] * torch.nn.functional.softplus(z[:, :na].float() + dt_bias).view(T, Hv, dk))
+    beta = torch.sigmoid(b.float())
+    gate = torch.sigmoid(z[:, na:].float()).view(T, Hv, dv)
+    for s in range(len(slot)):
+        r0, r1 = int(cu[s]), int(cu[s + 1])
+        if r1 <= r0:
+            continue
+        st = state[int(slot[s])]                                      # [Hv, dv, dk]
+        S = torch.zeros_like(st) if int(reset[s]) else st.clone()
+        for t in range(r0, r1):
+            S = S * g[t][:, None, :]
+            u = beta[t][:, None] * (v[t] - (S * k[t][:, None, :]).sum(-1))
+            S = S + u[:, :, None] * k[t][:, None, :]
+            o = (S * q[t][:, None, :]).sum(-1)
+            o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float() * gate[t]
+            out[t] = o.reshape(-1).to(out.dtype)
+        st.copy_(S)
+    return out
+
+
+def lightning_scan(q, k, v, decay, state, cu, slot, reset, out):
+    H, dv, dk = state.shape[1:]
+    T = q.shape[0]
+    silu = torch.nn.functional.silu
+    qf, kf, vf = silu(q.float()).view(T, H, dk), silu(k.float()).view(T, H, dk), silu(v.float()).view(T, H, dv)
+    for s in range(len(slot)):
+        r0, r1 = int(cu[s]), int(cu[s + 1])
+        if r1 <= r0:
+            continue
+        st = state[int(slot[s])]                                      # [H, dv, dk]
+        S = torch.zeros_like(st) if int(reset[s]) else st.clone()
+        for t in range(r0, r1):
+            S = S * decay[:, None, None] + vf[t][:, :, None] * kf[t][:, None, :]
+            out[t] = (S * qf[t][:, None, :]).sum(-1).reshape(-1).to(out.dtype)
+        st.copy_(S)
     return out
 
 
