@@ -7,18 +7,14 @@
 //       afterwards o / rms(o) * w * sigmoid(gate) per head
 //   lightning attention          S <- decay_h S + k_t v_t^T;  o_t = S^T q_t,   q, k, v = silu(projection)
 //
-// Prompt rows: `delta_prep` (parallel over rows: convolutions and unit norms, q / k in fp32), then
-// `state_scan` walks every sequence; `conv_tail` rewrites the convolution tails in a launch of its
-// own, because the rows before it read the old ones.  Single rows (decoding): `state_step`, one
+// Prompt rows run in chunks of 16: over a chunk the recurrence is a few small matrix products (for the
+// delta rule with a 16 x 16 triangular solve for the writes).  `chunk_prep` does everything that does not
+// need the state, parallel over (chunk, head): convolutions, unit norms, running decays, the 16 x 16
+// matrices, the decayed operands.  `chunk_scan` then walks the chunks of every (sequence, head) with the state
+// in MFMA accumulators, all products in fp32 (16 x 16 x 4).  `conv_tail` rewrites the convolution tails in a
+// launch of its own, because the rows before it read the old ones.  Single rows (decoding): `state_step`, one
 // launch from the projections to the normed, gated head output, tails included -- a workgroup owns
 // all heads that share a key head, so nobody else reads what it rewrites.
-//
-// Scan layout: column j of S (all key channels of one value channel) is spread over L = DKP / 8 lanes
-// of a wave, two groups of 4 neighbouring channels each (DKP: key width padded to 16 .. 512); the
-// dot products with k and q are in-lane sums and an L-lane DPP reduction, every lane carries NC
-// columns.  A workgroup takes 4 * (64 / L) * NC columns of one (sequence, head) and stages RB rows of
-// q, k, decays and values in LDS at a time: the next block's loads are in flight while the current one
-// runs, activations are applied once on the way into LDS, one barrier per block.
 #include "common.h"
 
 namespace {
@@ -71,155 +67,304 @@ __device__ __forceinline__ void ldn(const T* p, float (&f)[N]) {
 }
 
 // ------------------------------------------------------------------------------------------
-// convolutions + unit norms of prompt rows
+// prompt rows, in chunks of CH rows of a sequence (counted from its first row of the step)
 // ------------------------------------------------------------------------------------------
-struct PrepArgs {
-  int64_t stride;        // of the projection rows [q | k | v]
-  int C, K;              // convolved channels, taps
-  const int* first;      // [T] first row of the row's sequence in this step
-  const int* slot;       // [T] state slot, bit 30: the sequence starts in this step
-  float *qn, *kn, *qk;   // [T, Hk, DKP] x 2, [T, Hk]
-  int T, Hk, rep, dk, dv, DKP;
+constexpr int CH = 16;
+
+// grid row z -> (sequence, chunk of it); every wave scans the sequence lengths
+__device__ __forceinline__ bool find_chunk(const int* __restrict__ cu, int S, int z, int& s, int& c) {
+  const int lane = threadIdx.x & 63;
+  int before = 0;
+  for (int base = 0; base < S; base += 64) {
+    const int i = base + lane;
+    const int n = i < S ? (cu[i + 1] - cu[i] + CH - 1) / CH : 0;
+    int incl = n;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int t = __shfl_up(incl, o);
+      if (lane >= o) incl += t;
+    }
+    const int total = __shfl(incl, 63);
+    if (z < before + total) {
+      const unsigned long long m = __ballot(z < before + incl);
+      const int l = __ffsll(m) - 1;
+      s = base + l;
+      c = z - before - (__shfl(incl, l) - __shfl(n, l));
+      return true;
+    }
+    before += total;
+  }
+  return false;
+}
+// chunks of the sequences before s
+__device__ __forceinline__ int chunks_before(const int* __restrict__ cu, int s) {
+  int n = 0;
+  for (int i = threadIdx.x & 63; i < s; i += 64) n += (cu[i + 1] - cu[i] + CH - 1) / CH;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) n += __shfl_xor(n, o);
+  return n;
+}
+
+enum { DELTA = 0, LIGHTNING = 1 };
+
+// What `chunk_prep` leaves for `chunk_scan`, per (chunk, head), in floats: the operands of the state
+// products [CH][DKP] each (delta only: -G k), G q, the write keys transposed [DKP][CH], the state's decay over
+// the chunk [DKP], the CH x CH matrices (delta only: the solved write matrix), the read-out of the writes.
+template <int DKP, int MODE>
+struct ChunkLayout {
+  static constexpr int GK = 0, GQ = MODE == DELTA ? CH * DKP : 0, KT = GQ + CH * DKP, GC = KT + CH * DKP, TB = GC + DKP,
+                       BM = TB + (MODE == DELTA ? CH * CH : 0), SIZE = BM + CH * CH;
 };
 
-constexpr int PREP_ROWS = 4;   // rows per wave
+struct PrepArgs {
+  int64_t stride, z_stride, b_stride;   // rows of the projection (q, k, v / lightning: q, k), z, b
+  int K;                                // taps
+  const float *A_log, *dt_bias, *decay;
+  float* ws;                            // [chunks][H] chunk operands
+  const int *cu, *slot, *reset;
+  int S, H, Hk, dk, dv;
+};
 
-// SiLU(convolution) of channels ch .. ch + N - 1 at rows r .. r + PREP_ROWS - 1
-template <typename T, int N, int KT, bool VEC>
-__device__ __forceinline__ void conv_rows(const T* __restrict__ x, const T* __restrict__ w, const T* __restrict__ state,
-                                          const PrepArgs& a, int r, int ch, float (&y)[PREP_ROWS][N]) {
+// SiLU(convolution) of channels ch .. ch + N - 1 at rows r .. r + RW - 1 (clamped to `last`) of a sequence whose
+// step starts at row r0; st: the sequence's tail of channel ch, null when it starts in this step
+template <typename T, int N, int RW, int KT, bool VEC>
+__device__ __forceinline__ void conv_rows(const T* __restrict__ x, int64_t stride, const T* __restrict__ w,
+                                          const T* __restrict__ st, int K, int r0, int r, int last, int ch,
+                                          float (&y)[RW][N]) {
   if constexpr (KT > 0) {
-    float xs[PREP_ROWS + KT - 1][N], wt[KT][N];
+    float xs[RW + KT - 1][N], wt[KT][N];
 #pragma unroll
-    for (int i = 0; i < PREP_ROWS + KT - 1; ++i) {
-      const int rr = min(max(r - (KT - 1) + i, 0), a.T - 1);
-      ldn<T, N, VEC>(x + (int64_t)rr * a.stride + ch, xs[i]);
+    for (int i = 0; i < RW + KT - 1; ++i) {
+      const int rr = min(max(r - (KT - 1) + i, r0), last);
+      ldn<T, N, VEC>(x + (int64_t)rr * stride + ch, xs[i]);
     }
 #pragma unroll
     for (int n = 0; n < N; ++n)
 #pragma unroll
       for (int j = 0; j < KT; ++j) wt[j][n] = (float)w[(int64_t)(ch + n) * KT + j];
+    if (r - r0 < KT - 1) {      // rows before the step come from the tail
 #pragma unroll
-    for (int i = 0; i < PREP_ROWS; ++i) {
-      const int row = min(r + i, a.T - 1);
-      const int back = row - a.first[row];          // rows of the sequence before this one in the step
+      for (int i = 0; i < KT - 1; ++i) {
+        const int back = r0 - (r - (KT - 1) + i);   // this many rows before the step
+        if (back > 0) {
 #pragma unroll
-      for (int n = 0; n < N; ++n) y[i][n] = wt[KT - 1][n] * xs[i + KT - 1][n];
-      if (back >= KT - 1) {
-#pragma unroll
-        for (int j = 0; j < KT - 1; ++j)
-#pragma unroll
-          for (int n = 0; n < N; ++n) y[i][n] += wt[j][n] * xs[i + j][n];
-      } else {
-        const int sl = a.slot[row];
-        const bool fresh = (sl >> 30) & 1;
-        const T* st = state + ((int64_t)(sl & 0x3fffffff) * a.C + ch) * (KT - 1);
-#pragma unroll
-        for (int j = 0; j < KT - 1; ++j) {
-          const int d = KT - 1 - j;                 // tap j reads d rows back
-#pragma unroll
-          for (int n = 0; n < N; ++n) {
-            const float t = d <= back ? xs[i + j][n] : (fresh ? 0.f : (float)st[n * (KT - 1) + KT - 1 - (d - back)]);
-            y[i][n] += wt[j][n] * t;
-          }
+          for (int n = 0; n < N; ++n) xs[i][n] = st == nullptr ? 0.f : (float)st[n * (KT - 1) + KT - 1 - back];
         }
       }
-#pragma unroll
-      for (int n = 0; n < N; ++n) y[i][n] = silu<T>(y[i][n]);
     }
-  } else {
-    const int K = a.K;
-    for (int i = 0; i < PREP_ROWS; ++i) {
-      const int row = min(r + i, a.T - 1);
-      const int back = row - a.first[row], sl = a.slot[row];
-      const bool fresh = (sl >> 30) & 1;
+#pragma unroll
+    for (int i = 0; i < RW; ++i)
 #pragma unroll
       for (int n = 0; n < N; ++n) {
-        const T* st = state + ((int64_t)(sl & 0x3fffffff) * a.C + ch + n) * (K - 1);
         float acc = 0.f;
+#pragma unroll
+        for (int j = 0; j < KT; ++j) acc += wt[j][n] * xs[i + j][n];
+        y[i][n] = silu<T>(acc);
+      }
+  } else {
+#pragma unroll
+    for (int i = 0; i < RW; ++i)
+#pragma unroll
+      for (int n = 0; n < N; ++n) {
+        float acc = 0.f;
+        const int row = min(r + i, last);
         for (int j = 0; j < K; ++j) {
-          const int d = K - 1 - j;
-          const float t = d <= back ? (float)x[(int64_t)(row - d) * a.stride + ch + n]
-                                    : (fresh ? 0.f : (float)st[K - 1 - (d - back)]);
+          const int rr = row - (K - 1) + j;
+          const float t = rr >= r0 ? (float)x[(int64_t)rr * stride + ch + n]
+                                   : (st == nullptr ? 0.f : (float)st[n * (K - 1) + K - 1 - (r0 - rr)]);
           acc += (float)w[(int64_t)(ch + n) * K + j] * t;
         }
         y[i][n] = silu<T>(acc);
       }
-    }
   }
 }
 
-// One wave per (PREP_ROWS rows, key head): N channels of q and of k per lane (N * 64 >= DKP), then the
-// values of the head's `rep` value heads.
-template <typename T, int N, int KT, bool VEC>
-__global__ __launch_bounds__(256) void delta_prep_kernel(const T* __restrict__ x, const T* __restrict__ w,
-                                                         const T* __restrict__ state, T* __restrict__ v, PrepArgs a) {
-  const int lane = threadIdx.x & 63;
-  const int wid = blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int hk = wid % a.Hk, r = (wid / a.Hk) * PREP_ROWS;
-  if (r >= a.T) return;   // whole wave
-  const int c = lane * N, kd = a.Hk * a.dk;
-  float q[PREP_ROWS][N], k[PREP_ROWS][N];
+// One workgroup per (chunk, head).  N channels of q / k per lane (64 N >= DKP), four rows per wave.
+//   delta      A_ts = beta_t sum_c k_t k_s G_t / G_s (s < t);  the chunk's writes solve (1 + A) u = beta (v - (G k) S)
+//   both       B_ts = sum_c q_t k_s G_t / G_s (s <= t):        o = (G q) S + B u
+// with G_t the product of the decays from the chunk's start (ratios are powers of two of differences, which
+// never grow).  Rows beyond the sequence are empty: no key, no decay, nothing written.
+template <typename T, int DKP, int MODE, int KT, bool VEC>
+__global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x, const T* __restrict__ k_in,
+                                                         const T* __restrict__ w, const T* __restrict__ conv_state,
+                                                         const T* __restrict__ z, const T* __restrict__ b,
+                                                         T* __restrict__ v, PrepArgs a) {
+  constexpr int N = DKP > 64 ? DKP / 64 : 1, LD = DKP + 4, RW = CH / 4;
+  typedef ChunkLayout<DKP, MODE> Lay;
+  __shared__ __attribute__((aligned(16))) float sq[CH][LD], sk[CH][LD], sa[MODE == DELTA ? CH : 1][LD];
+  __shared__ __attribute__((aligned(16))) float sA[CH][CH + 4];
+  __shared__ float sb[CH + 1];
+  int s = 0, c = 0;
+  if (!find_chunk(a.cu, a.S, blockIdx.x, s, c)) return;   // uniform per block
+  const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int rep = a.H / a.Hk, hk = h / rep, dk = a.dk, dv = a.dv, kd = a.Hk * dk;
+  const int r0 = a.cu[s], r1 = a.cu[s + 1], ra = r0 + c * CH, nr = min(CH, r1 - ra), last = r1 - 1;
+  const int64_t slot = a.slot[s];
+  const bool fresh = a.reset[s] != 0;
+  float* ws = a.ws + ((int64_t)blockIdx.x * a.H + h) * Lay::SIZE;
+  const int ch0 = lane * N, row0 = wv * RW;
+
+  // ---- queries and keys of the wave's rows into LDS
+  float q[RW][N], k[RW][N];
 #pragma unroll
-  for (int i = 0; i < PREP_ROWS; ++i)
+  for (int i = 0; i < RW; ++i)
 #pragma unroll
     for (int n = 0; n < N; ++n) q[i][n] = k[i][n] = 0.f;
-  if (c + N <= a.dk) {
-    conv_rows<T, N, KT, VEC>(x, w, state, a, r, hk * a.dk + c, q);
-    conv_rows<T, N, KT, VEC>(x, w, state, a, r, kd + hk * a.dk + c, k);
-  } else if (N > 1) {
+  if constexpr (MODE == DELTA) {
+    const int C = 2 * kd + a.H * dv;
+    auto tail = [&](int ch) -> const T* { return fresh ? nullptr : conv_state + (slot * C + ch) * (a.K - 1); };
+    const int cq = hk * dk + ch0, ck = kd + cq;
+    if (row0 < nr) {
+      if (ch0 + N <= dk) {
+        conv_rows<T, N, RW, KT, VEC>(x, a.stride, w, tail(cq), a.K, r0, ra + row0, last, cq, q);
+        conv_rows<T, N, RW, KT, VEC>(x, a.stride, w, tail(ck), a.K, r0, ra + row0, last, ck, k);
+      } else if constexpr (N > 1) {
 #pragma unroll
-    for (int n = 0; n < N; ++n)
-      if (c + n < a.dk) {
-        float t[PREP_ROWS][1];
-        conv_rows<T, 1, KT, false>(x, w, state, a, r, hk * a.dk + c + n, t);
-        for (int i = 0; i < PREP_ROWS; ++i) q[i][n] = t[i][0];
-        conv_rows<T, 1, KT, false>(x, w, state, a, r, kd + hk * a.dk + c + n, t);
-        for (int i = 0; i < PREP_ROWS; ++i) k[i][n] = t[i][0];
+        for (int n = 0; n < N; ++n)
+          if (ch0 + n < dk) {
+            float t[RW][1];
+            conv_rows<T, 1, RW, KT, false>(x, a.stride, w, tail(cq + n), a.K, r0, ra + row0, last, cq + n, t);
+#pragma unroll
+            for (int i = 0; i < RW; ++i) q[i][n] = t[i][0];
+            conv_rows<T, 1, RW, KT, false>(x, a.stride, w, tail(ck + n), a.K, r0, ra + row0, last, ck + n, t);
+#pragma unroll
+            for (int i = 0; i < RW; ++i) k[i][n] = t[i][0];
+          }
       }
-  }
-  const float rd = 1.f / sqrtf((float)a.dk);
-#pragma unroll
-  for (int i = 0; i < PREP_ROWS; ++i) {
-    float sq = 0.f, sk = 0.f, sqk = 0.f;
-#pragma unroll
-    for (int n = 0; n < N; ++n) {
-      sq += q[i][n] * q[i][n];
-      sk += k[i][n] * k[i][n];
-      sqk += q[i][n] * k[i][n];
     }
-    sq = wave_sum(sq);
-    sk = wave_sum(sk);
-    sqk = wave_sum(sqk);
-    const float iq = rd / sqrtf(sq + 1e-6f), ik = 1.f / sqrtf(sk + 1e-6f);
-    if (r + i < a.T) {
-      const int64_t o = ((int64_t)(r + i) * a.Hk + hk);
-      if (c < a.DKP) {    // (N divides DKP: the padding is written as zeros)
-        float* qo = a.qn + o * a.DKP + c;
-        float* ko = a.kn + o * a.DKP + c;
+    const float rd = 1.f / sqrtf((float)dk);
 #pragma unroll
-        for (int n = 0; n < N; ++n) {
-          qo[n] = q[i][n] * iq;
-          ko[n] = k[i][n] * ik;
+    for (int i = 0; i < RW; ++i) {
+      float ssq = 0.f, ssk = 0.f;
+#pragma unroll
+      for (int n = 0; n < N; ++n) {
+        ssq += q[i][n] * q[i][n];
+        ssk += k[i][n] * k[i][n];
+      }
+      const float iq = rd / sqrtf(wave_sum(ssq) + 1e-6f), ik = 1.f / sqrtf(wave_sum(ssk) + 1e-6f);
+#pragma unroll
+      for (int n = 0; n < N; ++n) {
+        q[i][n] *= iq;
+        k[i][n] *= ik;
+      }
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < RW; ++i)
+#pragma unroll
+      for (int n = 0; n < N; ++n)
+        if (row0 + i < nr && ch0 + n < dk) {
+          const int64_t o = (int64_t)(ra + row0 + i) * a.stride + h * dk + ch0 + n;
+          q[i][n] = silu<T>((float)x[o]);
+          k[i][n] = silu<T>((float)k_in[o]);
         }
+  }
+  if (ch0 < DKP)
+#pragma unroll
+    for (int i = 0; i < RW; ++i)
+#pragma unroll
+      for (int n = 0; n < N; ++n) {
+        const bool on = row0 + i < nr;
+        sq[row0 + i][ch0 + n] = on ? q[i][n] : 0.f;
+        sk[row0 + i][ch0 + n] = on ? k[i][n] : 0.f;
       }
-      if (lane == 0) a.qk[o] = sqk * iq * ik;
+
+  // ---- decays (log2), write strengths, values
+  if constexpr (MODE == DELTA) {
+    const float A = expf(a.A_log[h]) * 1.44269504088896341f;
+    for (int e = tid; e < CH * DKP; e += 256) {
+      const int t = e / DKP, cc = e % DKP;
+      sa[t][cc] = t < nr && cc < dk
+                      ? -A * softplus((float)z[(int64_t)(ra + t) * a.z_stride + (int64_t)h * dk + cc] + a.dt_bias[(int64_t)h * dk + cc])
+                      : 0.f;
+    }
+    if (tid < CH) sb[tid] = tid < nr ? sigm<float>((float)b[(int64_t)(ra + tid) * a.b_stride + h]) : 0.f;
+    constexpr int NV = VEC ? 2 : 1;
+    const int C = 2 * kd + a.H * dv;
+    for (int cv = lane * NV; cv < dv && row0 < nr; cv += 64 * NV) {
+      const int ch = 2 * kd + h * dv + cv;
+      float t[RW][NV];
+      conv_rows<T, NV, RW, KT, VEC>(x, a.stride, w, fresh ? nullptr : conv_state + (slot * C + ch) * (a.K - 1), a.K, r0,
+                                    ra + row0, last, ch, t);
+#pragma unroll
+      for (int i = 0; i < RW; ++i)
+        if (row0 + i < nr) {
+          T* vo = v + ((int64_t)(ra + row0 + i) * a.H + h) * dv + cv;
+#pragma unroll
+          for (int n = 0; n < NV; ++n) vo[n] = (T)t[i][n];
+        }
+    }
+    __syncthreads();
+    for (int cc = tid; cc < DKP; cc += 256) {   // running sums over the chunk
+      float acc = 0.f;
+#pragma unroll
+      for (int t = 0; t < CH; ++t) {
+        acc += sa[t][cc];
+        sa[t][cc] = acc;
+      }
+    }
+  } else {
+    if (tid <= CH) sb[tid] = powf(a.decay[h], (float)tid);
+  }
+  __syncthreads();
+
+  // ---- the CH x CH products, one pair of rows per thread
+  {
+    const int t = tid / CH, u = tid % CH;
+    float kk = 0.f, qk = 0.f;
+#pragma unroll 4
+    for (int cc = 0; cc < DKP; cc += 4) {
+      const f32x4 ku = *reinterpret_cast<const f32x4*>(&sk[u][cc]), qt = *reinterpret_cast<const f32x4*>(&sq[t][cc]);
+      if constexpr (MODE == DELTA) {
+        const f32x4 kt = *reinterpret_cast<const f32x4*>(&sk[t][cc]);
+        const f32x4 at = *reinterpret_cast<const f32x4*>(&sa[t][cc]), au = *reinterpret_cast<const f32x4*>(&sa[u][cc]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float f = ku[e] * __builtin_amdgcn_exp2f(fminf(at[e] - au[e], 0.f));   // (pairs u > t are dropped below)
+          kk += kt[e] * f;
+          qk += qt[e] * f;
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) qk += qt[e] * ku[e];
+      }
+    }
+    if constexpr (MODE == DELTA) {
+      sA[t][u] = u < t ? sb[t] * kk : 0.f;
+      ws[Lay::BM + tid] = u <= t ? qk : 0.f;
+    } else {
+      ws[Lay::BM + tid] = u <= t ? qk * sb[t - u] : 0.f;
     }
   }
-  // values: rep * dv channels of the group, two per lane where that divides
-  const int nv = a.rep * a.dv, v0 = hk * nv, VD = a.Hk * nv;
-  constexpr int NV = VEC ? 2 : 1;
-  for (int cv = lane * NV; cv < nv; cv += 64 * NV) {
-    float t[PREP_ROWS][NV];
-    conv_rows<T, NV, KT, VEC>(x, w, state, a, r, 2 * kd + v0 + cv, t);
+  if constexpr (MODE == DELTA) {
+    __syncthreads();
+    if (wv == 0) {   // X = (1 + A)^-1 column by column; the write matrix is X diag(beta)
+      float X[CH];
 #pragma unroll
-    for (int i = 0; i < PREP_ROWS; ++i)
-      if (r + i < a.T) {
-        T* vo = v + (int64_t)(r + i) * VD + v0 + cv;
+      for (int t = 0; t < CH; ++t) {
+        float acc = t == lane ? 1.f : 0.f;
 #pragma unroll
-        for (int n = 0; n < NV; ++n) vo[n] = (T)t[i][n];
+        for (int u = 0; u < t; ++u) acc -= sA[t][u] * X[u];
+        X[t] = acc;
       }
+      if (lane < CH)
+#pragma unroll
+        for (int t = 0; t < CH; ++t) ws[Lay::TB + t * CH + lane] = X[t] * sb[lane];
+    }
   }
+  // ---- operands of the state products
+  for (int e = tid; e < CH * DKP; e += 256) {
+    const int t = e / DKP, cc = e % DKP;
+    const float g = MODE == DELTA ? __builtin_amdgcn_exp2f(sa[t][cc]) : sb[min(t + 1, nr)];
+    if constexpr (MODE == DELTA) ws[Lay::GK + e] = -g * sk[t][cc];
+    ws[Lay::GQ + e] = g * sq[t][cc];
+  }
+  for (int e = tid; e < CH * DKP; e += 256) {
+    const int cc = e / CH, t = e % CH;
+    const float g = MODE == DELTA ? __builtin_amdgcn_exp2f(sa[CH - 1][cc] - sa[t][cc]) : sb[max(nr - 1 - t, 0)];
+    ws[Lay::KT + e] = g * sk[t][cc];
+  }
+  for (int cc = tid; cc < DKP; cc += 256) ws[Lay::GC + cc] = MODE == DELTA ? __builtin_amdgcn_exp2f(sa[CH - 1][cc]) : sb[nr];
 }
 
 // state[slot][c][j] <- the raw input of the j-th of a sequence's last K - 1 rows
@@ -239,201 +384,157 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ x,
   }
 }
 
-// ------------------------------------------------------------------------------------------
-// scan
-// ------------------------------------------------------------------------------------------
 struct ScanArgs {
-  const float *qn, *kn, *qk;          // delta: [T, Hk, DKP] x 2, [T, Hk]
-  int64_t q_stride, v_stride;         // lightning: rows of the projection (q, k, v); delta: rows of v
-  const float *A_log, *dt_bias;       // delta: [H], [H * dk]
-  int64_t z_stride, b_stride;
-  const float* decay;                 // lightning: [H]
+  const float* ws;
+  int64_t v_stride;
   float* state;
   const int *cu, *slot, *reset;
-  int H, Hk, dk, dv;
+  int H, dk, dv;
 };
 
-enum { DELTA = 0, LIGHTNING = 1 };
+__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
 
-template <typename T, int L, int NC, int MODE, int RB>
-__global__ __launch_bounds__(256) void state_scan_kernel(const T* __restrict__ q, const T* __restrict__ k,
-                                                         const T* __restrict__ v, const T* __restrict__ z,
-                                                         const T* __restrict__ b, T* __restrict__ out, ScanArgs a) {
-  constexpr int DKP = 8 * L, GPW = 64 / L, CPB = 4 * GPW * NC;
-  constexpr int NK = (RB * DKP + 255) / 256, NV = (RB * CPB + 255) / 256;   // staged elements per thread
-  constexpr int ROWF = (MODE == DELTA ? 3 : 2) * DKP + CPB + 4;             // floats of a staged row
-  __shared__ __attribute__((aligned(16))) float sm[2][RB][ROWF];
-  const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+// Walks the chunks of one (sequence, head); wave w owns 16 value columns.  Accumulator layout of the
+// 16 x 16 x 4 product: lane (g = lane / 16, li = lane % 16) holds rows 4 g + r of column li; as the second
+// operand lane (g, li) supplies row g.  The order of a dot product's terms is free, so product r of a tile takes
+// the rows {4 g + r}: an accumulator's element r IS the second operand, and the first operand's four elements
+// are neighbours in LDS.  The state (channels 16 m + 4 g + r of column li) never leaves its accumulators.
+template <typename T, int DKP, int MODE, int NBUF>
+__global__ __launch_bounds__(256) void chunk_scan_kernel(const T* __restrict__ v, T* __restrict__ out, ScanArgs a) {
+  typedef ChunkLayout<DKP, MODE> Lay;
+  constexpr int M = DKP / 16, LD = DKP + 4, LT = CH + 4;
+  constexpr int OGK = 0, OGQ = MODE == DELTA ? CH * LD : 0, OKT = OGQ + CH * LD, OGC = OKT + DKP * LT, OTB = OGC + DKP,
+                OBM = OTB + (MODE == DELTA ? CH * LT : 0), OSZ = OBM + CH * LT;   // the same operands with padded rows
+  constexpr int NF = (Lay::SIZE / 4 + 255) / 256;   // 16-byte loads per thread and chunk
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, g = lane >> 4, li = lane & 15;
   const int r0 = a.cu[s], r1 = a.cu[s + 1];
   if (r1 <= r0) return;   // uniform per block
-  const int lane = tid & 63, wv = tid >> 6, li = lane % L;
-  const int cb = blockIdx.z * CPB, cl = (wv * GPW + lane / L) * NC;   // the block's / the lane's first column
-  const int hk = h / (a.H / a.Hk), dk = a.dk, dv = a.dv;
+  const int col = blockIdx.z * 64 + (tid >> 6) * 16 + li, dk = a.dk, dv = a.dv;
+  const bool on = col < dv;
+  float* st = a.state + (((int64_t)a.slot[s] * a.H + h) * dv + (on ? col : 0)) * dk;
+  const bool vec = dk % 4 == 0;
+  f32x4 S[M];
   const bool fresh = a.reset[s] != 0;
-  float* st = a.state + ((int64_t)a.slot[s] * a.H + h) * dv * dk;
-  const bool vec = dk == DKP;
-  f32x4 S0[NC], S1[NC];
 #pragma unroll
-  for (int c = 0; c < NC; ++c) {
-    S0[c] = S1[c] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (!fresh && cb + cl + c < dv) {
-      const float* p = st + (int64_t)(cb + cl + c) * dk;
-      if (vec) {
-        S0[c] = *reinterpret_cast<const f32x4*>(p + 4 * li);
-        S1[c] = *reinterpret_cast<const f32x4*>(p + 4 * (L + li));
-      } else {
+  for (int m = 0; m < M; ++m) {
+    S[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int c = 16 * m + 4 * g;
+    if (on && !fresh && c < dk) {
+      if (vec) S[m] = *reinterpret_cast<const f32x4*>(st + c);
+      else
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          S0[c][e] = 4 * li + e < dk ? p[4 * li + e] : 0.f;
-          S1[c][e] = 4 * (L + li) + e < dk ? p[4 * (L + li) + e] : 0.f;
-        }
-      }
+        for (int r = 0; r < 4; ++r) S[m][r] = c + r < dk ? st[c + r] : 0.f;
     }
   }
-  const float A = MODE == DELTA ? expf(a.A_log[h]) : 0.f;
-  const float dec = MODE == LIGHTNING ? a.decay[h] : 0.f;
-
-  // raw operands of the rows rb .. rb + RB - 1 (addresses clamped to the sequence and the head)
-  float rq[NK], rk[NK], rz[MODE == DELTA ? NK : 1], rv[NV], rs = 0.f;
-  auto fetch = [&](int rb) {
+  const int nc = (r1 - r0 + CH - 1) / CH;
+  const float* ws = a.ws + ((int64_t)chunks_before(a.cu, s) * a.H + h) * Lay::SIZE;
+  f32x4 pre[NF], pv;
+  auto fetch = [&](int c) {
+    const f32x4* p = reinterpret_cast<const f32x4*>(ws + (int64_t)c * a.H * Lay::SIZE);
 #pragma unroll
-    for (int u = 0; u < NK; ++u) {
-      const int e = tid + 256 * u, r = min(rb + e / DKP, r1 - 1), c = e % DKP;
-      if constexpr (MODE == DELTA) {
-        const int64_t o = ((int64_t)r * a.Hk + hk) * DKP + c;
-        rq[u] = a.qn[o];
-        rk[u] = a.kn[o];
-        rz[u] = (float)z[(int64_t)r * a.z_stride + (int64_t)h * dk + min(c, dk - 1)];
-      } else {
-        const int64_t o = (int64_t)r * a.q_stride + (int64_t)hk * dk + min(c, dk - 1);
-        rq[u] = (float)q[o];
-        rk[u] = (float)k[o];
+    for (int u = 0; u < NF; ++u)
+      if (tid + 256 * u < Lay::SIZE / 4) pre[u] = p[tid + 256 * u];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = r0 + c * CH + 4 * g + r;
+      float t = 0.f;
+      if (on && row < r1) {
+        t = (float)v[(int64_t)row * a.v_stride + (int64_t)h * dv + col];
+        if constexpr (MODE == LIGHTNING) t = silu<T>(t);
       }
-    }
-#pragma unroll
-    for (int u = 0; u < NV; ++u) {
-      const int e = tid + 256 * u, r = min(rb + e / CPB, r1 - 1), c = min(cb + e % CPB, dv - 1);
-      rv[u] = (float)v[(int64_t)r * a.v_stride + (int64_t)h * dv + c];
-    }
-    if (MODE == DELTA && tid < 2 * RB) {
-      const int r = min(rb + tid / 2, r1 - 1);
-      rs = tid & 1 ? a.qk[(int64_t)r * a.Hk + hk] : (float)b[(int64_t)r * a.b_stride + h];
+      pv[r] = t;
     }
   };
-  float db[MODE == DELTA ? NK : 1];
-  if constexpr (MODE == DELTA) {
+  auto store = [&](float* p) {
 #pragma unroll
-    for (int u = 0; u < NK; ++u) db[u] = a.dt_bias[(int64_t)h * dk + min((tid + 256 * u) % DKP, dk - 1)];
-  }
-  auto store = [&](int p) {
-#pragma unroll
-    for (int u = 0; u < NK; ++u) {
-      const int e = tid + 256 * u, r = e / DKP, c = e % DKP;
-      if (RB * DKP % 256 == 0 || e < RB * DKP) {
-        if constexpr (MODE == DELTA) {
-          sm[p][r][c] = rq[u];
-          sm[p][r][DKP + c] = rk[u];
-          sm[p][r][2 * DKP + c] = decay_of(rz[u], db[u], A);
-        } else {
-          sm[p][r][c] = c < dk ? silu<T>(rq[u]) : 0.f;
-          sm[p][r][DKP + c] = c < dk ? silu<T>(rk[u]) : 0.f;
-        }
-      }
+    for (int u = 0; u < NF; ++u) {
+      const int e = 4 * (tid + 256 * u);
+      if (e >= Lay::SIZE) continue;
+      int o;
+      if (MODE == DELTA && e < Lay::GQ) o = OGK + e / DKP * LD + e % DKP;
+      else if (e < Lay::KT) o = OGQ + (e - Lay::GQ) / DKP * LD + (e - Lay::GQ) % DKP;
+      else if (e < Lay::GC) o = OKT + (e - Lay::KT) / CH * LT + (e - Lay::KT) % CH;
+      else if (e < Lay::TB) o = OGC + e - Lay::GC;
+      else if (e < Lay::BM) o = OTB + (e - Lay::TB) / CH * LT + (e - Lay::TB) % CH;
+      else o = OBM + (e - Lay::BM) / CH * LT + (e - Lay::BM) % CH;
+      *reinterpret_cast<f32x4*>(p + o) = pre[u];
     }
-    constexpr int VO = (MODE == DELTA ? 3 : 2) * DKP;
-#pragma unroll
-    for (int u = 0; u < NV; ++u) {
-      const int e = tid + 256 * u;
-      if (RB * CPB % 256 == 0 || e < RB * CPB) sm[p][e / CPB][VO + e % CPB] = MODE == LIGHTNING ? silu<T>(rv[u]) : rv[u];
-    }
-    if (MODE == DELTA && tid < 2 * RB) sm[p][tid / 2][VO + CPB + (tid & 1)] = tid & 1 ? rs : sigm<float>(rs);
   };
-
-  fetch(r0);
-  store(0);
-  __syncthreads();
-  int p = 0;
-  for (int rb = r0; rb < r1; rb += RB, p ^= 1) {
-    const bool more = rb + RB < r1;
-    if (more) fetch(rb + RB);
-    const int nb = min(RB, r1 - rb);
-#pragma unroll 2
-    for (int t = 0; t < nb; ++t) {
-      const float* row = sm[p][t];
-      const f32x4 q0 = *reinterpret_cast<const f32x4*>(row + 4 * li), q1 = *reinterpret_cast<const f32x4*>(row + 4 * (L + li));
-      const f32x4 k0 = *reinterpret_cast<const f32x4*>(row + DKP + 4 * li),
-                  k1 = *reinterpret_cast<const f32x4*>(row + DKP + 4 * (L + li));
-      constexpr int VO = (MODE == DELTA ? 3 : 2) * DKP;
-      float vj[NC], o[NC];
+  auto rd4 = [](const float* p) { return *reinterpret_cast<const f32x4*>(p); };
+  fetch(0);
+  int buf = 0;
+  for (int c = 0; c < nc; ++c) {
+    float* p = sm + buf * OSZ;
+    if (NBUF == 1 && c > 0) __syncthreads();   // the previous chunk's readers
+    store(p);
+    f32x4 R = pv, O = f32x4{0.f, 0.f, 0.f, 0.f};
+    __syncthreads();    // (two buffers: the one written next was last read before this barrier)
+    if (c + 1 < nc) fetch(c + 1);
+    if constexpr (MODE == DELTA) {
 #pragma unroll
-      for (int c = 0; c < NC; ++c) vj[c] = row[VO + cl + c];
-      if constexpr (MODE == DELTA) {
-        const f32x4 g0 = *reinterpret_cast<const f32x4*>(row + 2 * DKP + 4 * li),
-                    g1 = *reinterpret_cast<const f32x4*>(row + 2 * DKP + 4 * (L + li));
-        const float beta = row[VO + CPB], kq = row[VO + CPB + 1];
-        float sk[NC], sq[NC];
+      for (int m = 0; m < M; ++m) {
+        const f32x4 gk = rd4(p + OGK + li * LD + 16 * m + 4 * g), gq = rd4(p + OGQ + li * LD + 16 * m + 4 * g);
 #pragma unroll
-        for (int c = 0; c < NC; ++c) {
-          sk[c] = sq[c] = 0.f;
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            S0[c][e] *= g0[e];
-            S1[c][e] *= g1[e];
-            sk[c] += S0[c][e] * k0[e] + S1[c][e] * k1[e];
-            sq[c] += S0[c][e] * q0[e] + S1[c][e] * q1[e];
-          }
+        for (int r = 0; r < 4; ++r) {
+          R = mfma4(gk[r], S[m][r], R);
+          O = mfma4(gq[r], S[m][r], O);
         }
-#pragma unroll
-        for (int c = 0; c < NC; ++c) {
-          sk[c] = lanes_sum<L>(sk[c]);
-          sq[c] = lanes_sum<L>(sq[c]);
-        }
-#pragma unroll
-        for (int c = 0; c < NC; ++c) {
-          const float u = (vj[c] - sk[c]) * beta;
-          o[c] = sq[c] + u * kq;
-          S0[c] += k0 * u;
-          S1[c] += k1 * u;
-        }
-      } else {
-#pragma unroll
-        for (int c = 0; c < NC; ++c) {
-          o[c] = 0.f;
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            S0[c][e] = S0[c][e] * dec + k0[e] * vj[c];
-            S1[c][e] = S1[c][e] * dec + k1[e] * vj[c];
-            o[c] += S0[c][e] * q0[e] + S1[c][e] * q1[e];
-          }
-        }
-#pragma unroll
-        for (int c = 0; c < NC; ++c) o[c] = lanes_sum<L>(o[c]);
       }
-      if (li == 0) {
-        T* oo = out + (int64_t)(rb + t) * a.H * dv + (int64_t)h * dv + cb + cl;
+      const f32x4 tb = rd4(p + OTB + li * LT + 4 * g);
+      f32x4 U = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int c = 0; c < NC; ++c)
-          if (cb + cl + c < dv) oo[c] = (T)o[c];
+      for (int r = 0; r < 4; ++r) U = mfma4(tb[r], R[r], U);
+      R = U;
+    } else {
+      f32x4 O2 = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int m = 0; m < M; ++m) {
+        const f32x4 gq = rd4(p + OGQ + li * LD + 16 * m + 4 * g);
+#pragma unroll
+        for (int r = 0; r < 4; r += 2) {
+          O = mfma4(gq[r], S[m][r], O);
+          O2 = mfma4(gq[r + 1], S[m][r + 1], O2);
+        }
+      }
+      O += O2;
+    }
+#pragma unroll
+    for (int m = 0; m < M; ++m) S[m] *= rd4(p + OGC + 16 * m + 4 * g);
+    const f32x4 bm = rd4(p + OBM + li * LT + 4 * g);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) O = mfma4(bm[r], R[r], O);
+#pragma unroll
+    for (int m = 0; m < M; m += 2) {
+      const f32x4 k0 = rd4(p + OKT + (16 * m + li) * LT + 4 * g);
+      const f32x4 k1 = M > 1 ? rd4(p + OKT + (16 * (m + (M > 1)) + li) * LT + 4 * g) : k0;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        S[m] = mfma4(k0[r], R[r], S[m]);
+        if constexpr (M > 1) S[m + 1] = mfma4(k1[r], R[r], S[m + 1]);
       }
     }
-    if (more) store(p ^ 1);   // (last read before the previous barrier)
-    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = r0 + c * CH + 4 * g + r;
+      if (on && row < r1) out[((int64_t)row * a.H + h) * dv + col] = (T)O[r];
+    }
+    if constexpr (NBUF == 2) buf ^= 1;
   }
+  if (!on) return;
 #pragma unroll
-  for (int c = 0; c < NC; ++c)
-    if (cb + cl + c < dv) {
-      float* w = st + (int64_t)(cb + cl + c) * dk;
-      if (vec) {
-        *reinterpret_cast<f32x4*>(w + 4 * li) = S0[c];
-        *reinterpret_cast<f32x4*>(w + 4 * (L + li)) = S1[c];
-      } else {
+  for (int m = 0; m < M; ++m) {
+    const int c = 16 * m + 4 * g;
+    if (c < dk) {
+      if (vec) *reinterpret_cast<f32x4*>(st + c) = S[m];
+      else
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          if (4 * li + e < dk) w[4 * li + e] = S0[c][e];
-          if (4 * (L + li) + e < dk) w[4 * (L + li) + e] = S1[c][e];
-        }
-      }
+        for (int r = 0; r < 4; ++r)
+          if (c + r < dk) st[c + r] = S[m][r];
     }
+  }
 }
 
 // ------------------------------------------------------------------------------------------
@@ -652,53 +753,51 @@ int padded_dk(int dk) {
   return p;
 }
 
-template <typename T, int N, bool VEC>
-int prep(const void* x, const void* w, const void* state, void* v, const PrepArgs& a, hipStream_t stream) {
-  const int64_t waves = (int64_t)((a.T + PREP_ROWS - 1) / PREP_ROWS) * a.Hk;
-  const int nblk = (int)((waves + 3) / 4);
-#define PREP(KT) \
-  delta_prep_kernel<T, N, KT, VEC><<<nblk, 256, 0, stream>>>((const T*)x, (const T*)w, (const T*)state, (T*)v, a)
-  if (a.K == 2) PREP(2);
-  else if (a.K == 3) PREP(3);
-  else if (a.K == 4) PREP(4);
-  else PREP(0);
+template <typename T, int DKP, int MODE>
+int chunked(const void* x, const void* k, const void* v_in, const void* w, const void* conv_state, const void* z, const void* b,
+            void* v, const PrepArgs& p, const ScanArgs& a, void* out, int chunks, bool vec, hipStream_t stream) {
+  typedef ChunkLayout<DKP, MODE> Lay;
+  const dim3 pg(chunks, p.H);
+#define PREP(KT, V)                                                                                             \
+  chunk_prep_kernel<T, DKP, MODE, KT, V><<<pg, 256, 0, stream>>>((const T*)x, (const T*)k, (const T*)w,        \
+                                                                 (const T*)conv_state, (const T*)z, (const T*)b, (T*)v, p)
+  if constexpr (MODE == LIGHTNING) {
+    PREP(0, false);
+  } else if (vec) {
+    if (p.K == 2) PREP(2, true);
+    else if (p.K == 3) PREP(3, true);
+    else if (p.K == 4) PREP(4, true);
+    else PREP(0, true);
+  } else {
+    if (p.K == 2) PREP(2, false);
+    else if (p.K == 3) PREP(3, false);
+    else if (p.K == 4) PREP(4, false);
+    else PREP(0, false);
+  }
 #undef PREP
   OME_CHECK_LAUNCH();
-  return 0;
-}
-
-template <typename T, int L, int MODE>
-int scan(const void* q, const void* k, const void* v, const void* z, const void* b, void* out, const ScanArgs& a, int S,
-         int nc, hipStream_t stream) {
-  constexpr int RB = L <= 16 ? 8 : (L == 32 ? 4 : 2), GPW = 64 / L;
-  const dim3 grid(S, a.H, (a.dv + 4 * GPW * nc - 1) / (4 * GPW * nc));
-#define SCAN(NC)                                                                                                  \
-  state_scan_kernel<T, L, NC, MODE, RB><<<grid, 256, 0, stream>>>((const T*)q, (const T*)k, (const T*)v, (const T*)z, \
-                                                                  (const T*)b, (T*)out, a)
-  if (nc == 1) SCAN(1);
-  else if (nc == 2) SCAN(2);
-  else SCAN(4);
-#undef SCAN
+  constexpr int LD = DKP + 4, LT = CH + 4, NBUF = DKP <= 128 ? 2 : 1;
+  constexpr int lds = NBUF * ((MODE == DELTA ? 2 : 1) * CH * LD + DKP * LT + DKP + (MODE == DELTA ? 2 : 1) * CH * LT) * 4;
+  static_assert(lds <= 64 * 1024 && Lay::SIZE % 4 == 0, "chunk operands in LDS");
+  const dim3 sg(p.S, p.H, (p.dv + 63) / 64);
+  chunk_scan_kernel<T, DKP, MODE, NBUF><<<sg, 256, lds, stream>>>((const T*)v_in, (T*)out, a);
   OME_CHECK_LAUNCH();
   return 0;
 }
 
 template <typename T, int MODE>
-int scan_by_width(const void* q, const void* k, const void* v, const void* z, const void* b, void* out, const ScanArgs& a,
-                  int S, hipStream_t stream) {
-  const int DKP = padded_dk(a.dk), gpw = 64 / (DKP / 8);
-  // columns per lane: more of them share a row's operands, fewer leave more workgroups
-  int nc = 4;
-  while (nc > 1 && (int64_t)S * a.H * ((a.dv + 4 * gpw * nc - 1) / (4 * gpw * nc)) < 512) nc /= 2;
-  while (nc > 1 && 4 * gpw * (nc / 2) >= a.dv) nc /= 2;
-  switch (DKP) {
-    case 16: return scan<T, 2, MODE>(q, k, v, z, b, out, a, S, nc, stream);
-    case 32: return scan<T, 4, MODE>(q, k, v, z, b, out, a, S, nc, stream);
-    case 64: return scan<T, 8, MODE>(q, k, v, z, b, out, a, S, nc, stream);
-    case 128: return scan<T, 16, MODE>(q, k, v, z, b, out, a, S, nc, stream);
-    case 256: return scan<T, 32, MODE>(q, k, v, z, b, out, a, S, nc, stream);
-    default: return scan<T, 64, MODE>(q, k, v, z, b, out, a, S, nc, stream);
+int chunked_by_width(const void* x, const void* k, const void* v_in, const void* w, const void* conv_state, const void* z,
+                     const void* b, void* v, const PrepArgs& p, const ScanArgs& a, void* out, int chunks, bool vec,
+                     hipStream_t stream) {
+#define GO(D) chunked<T, D, MODE>(x, k, v_in, w, conv_state, z, b, v, p, a, out, chunks, vec, stream)
+  switch (padded_dk(p.dk)) {
+    case 16: return GO(16);
+    case 32: return GO(32);
+    case 64: return GO(64);
+    case 128: return GO(128);
+    default: return GO(256);
   }
+#undef GO
 }
 
 template <typename T, int MODE>
@@ -717,44 +816,18 @@ int step_by_width(const void* q, const void* k, const void* v, const void* conv_
     case 32: STEP(4); break;
     case 64: STEP(8); break;
     case 128: STEP(16); break;
-    case 256: STEP(32); break;
-    default: STEP(64); break;
+    default: STEP(32); break;
   }
 #undef STEP
   OME_CHECK_LAUNCH();
   return 0;
 }
 
-bool bad_shape(int H, int Hk, int dk, int dv) { return Hk <= 0 || H <= 0 || H % Hk || dk <= 0 || dk > 512 || dv <= 0; }
+bool bad_shape(int S, int H, int Hk, int dk, int dv) {
+  return Hk <= 0 || H <= 0 || H % Hk || dk <= 0 || dk > 256 || dv <= 0 || H > 65535 || S > 0x7fffffff / 64;
+}
 
 }  // namespace
-
-// x: projection rows [q (Hk * dk) | k (Hk * dk) | v (H * dv)] (row stride in elements), conv_w [C, K], conv_state
-// [slots, C, K - 1]; first / slot [T]: see PrepArgs; qn / kn fp32 [T, Hk, DKP], qk fp32 [T, Hk], v [T, H * dv].
-OME_API int ome_delta_prep(const void* x, int64_t stride, const void* conv_w, const void* conv_state, int K,
-                           const int* first, const int* slot, float* qn, float* kn, float* qk, void* v, int T, int H,
-                           int Hk, int dk, int dv, int f32, hipStream_t stream) {
-  if (T <= 0) return 0;
-  if (bad_shape(H, Hk, dk, dv) || K < 1 || K > 32) return -2;
-  const int DKP = padded_dk(dk);
-  const PrepArgs a{stride, 2 * Hk * dk + H * dv, K, first, slot, qn, kn, qk, T, Hk, H / Hk, dk, dv, DKP};
-  const int esz = f32 ? 4 : 2;
-  const int N = DKP <= 64 ? 1 : DKP / 64;
-  const int A = N > 2 ? N : 2;   // elements a vector access needs aligned
-  const bool vec = N > 1 && dk % A == 0 && (H / Hk * dv) % 2 == 0 && stride % A == 0 && ((uintptr_t)x & (A * esz - 1)) == 0;
-#define PREP_N(TT, NN) (vec ? prep<TT, NN, true>(x, conv_w, conv_state, v, a, stream) : prep<TT, NN, false>(x, conv_w, conv_state, v, a, stream))
-  if (f32) {
-    if (N == 1) return prep<float, 1, false>(x, conv_w, conv_state, v, a, stream);
-    if (N == 2) return PREP_N(float, 2);
-    if (N == 4) return PREP_N(float, 4);
-    return prep<float, 8, false>(x, conv_w, conv_state, v, a, stream);
-  }
-  if (N == 1) return prep<bf16, 1, false>(x, conv_w, conv_state, v, a, stream);
-  if (N == 2) return PREP_N(bf16, 2);
-  if (N == 4) return PREP_N(bf16, 4);
-  return PREP_N(bf16, 8);
-#undef PREP_N
-}
 
 OME_API int ome_conv_tail(const void* x, int64_t stride, void* state, const int* cu, const int* slot, const int* reset,
                           int S, int C, int K, int f32, hipStream_t stream) {
@@ -767,28 +840,41 @@ OME_API int ome_conv_tail(const void* x, int64_t stride, void* state, const int*
   return 0;
 }
 
-// Delta rule over the rows of every sequence: operands of ome_delta_prep, z rows [decay inputs (H * dk) | ..], b rows
-// [H]; state fp32 [slots, H, dv, dk]; out [T, H * dv] (before the head norm).
-OME_API int ome_delta_scan(const float* qn, const float* kn, const float* qk, const void* v, const void* z,
-                           int64_t z_stride, const void* b, int64_t b_stride, const float* A_log, const float* dt_bias,
-                           float* state, void* out, const int* cu, const int* slot, const int* reset, int S, int H, int Hk,
-                           int dk, int dv, int f32, hipStream_t stream) {
-  if (S <= 0) return 0;
-  if (bad_shape(H, Hk, dk, dv) || H > 65535) return -2;
-  const ScanArgs a{qn, kn, qk, 0, (int64_t)H * dv, A_log, dt_bias, z_stride, b_stride, nullptr, state, cu, slot, reset, H, Hk, dk, dv};
-  if (f32) return scan_by_width<float, DELTA>(nullptr, nullptr, v, z, b, out, a, S, stream);
-  return scan_by_width<bf16, DELTA>(nullptr, nullptr, v, z, b, out, a, S, stream);
+// floats of workspace per (chunk of 16 rows, head)
+OME_API int ome_state_chunk_floats(int dk, int delta) {
+  const int DKP = padded_dk(dk);
+  return (delta ? 3 : 2) * CH * DKP + DKP + (delta ? 2 : 1) * CH * CH;
+}
+
+// Delta rule over the rows of every sequence.  x: projection rows [q (Hk * dk) | k (Hk * dk) | v (H * dv)] (row stride in
+// elements), conv_w [C, K], conv_state [slots, C, K - 1]; z rows [decay inputs (H * dk) | ..], b rows [H]; v: scratch
+// [T, H * dv]; ws: ome_state_chunk_floats per (chunk, head), chunks >= sum over sequences of ceil(rows / 16);
+// state fp32 [slots, H, dv, dk]; out [T, H * dv] (before the head norm).
+OME_API int ome_delta_scan(const void* x, int64_t stride, const void* conv_w, const void* conv_state, int K, const void* z,
+                           int64_t z_stride, const void* b, int64_t b_stride, const float* A_log, const float* dt_bias, void* v,
+                           float* ws, int chunks, float* state, void* out, const int* cu, const int* slot, const int* reset,
+                           int S, int H, int Hk, int dk, int dv, int f32, hipStream_t stream) {
+  if (S <= 0 || chunks <= 0) return 0;
+  if (bad_shape(S, H, Hk, dk, dv) || K < 1 || K > 32) return -2;
+  const PrepArgs p{stride, z_stride, b_stride, K, A_log, dt_bias, nullptr, ws, cu, slot, reset, S, H, Hk, dk, dv};
+  const ScanArgs a{ws, (int64_t)H * dv, state, cu, slot, reset, H, dk, dv};
+  const int N = padded_dk(dk) > 64 ? padded_dk(dk) / 64 : 1, A = N > 2 ? N : 2;   // elements a vector access needs aligned
+  const bool vec = N > 1 && dk % A == 0 && dv % 2 == 0 && stride % A == 0 && ((uintptr_t)x & (A * (f32 ? 4 : 2) - 1)) == 0;
+  if (f32) return chunked_by_width<float, DELTA>(x, nullptr, v, conv_w, conv_state, z, b, v, p, a, out, chunks, vec, stream);
+  return chunked_by_width<bf16, DELTA>(x, nullptr, v, conv_w, conv_state, z, b, v, p, a, out, chunks, vec, stream);
 }
 
 // q / k [T, H * dk], v [T, H * dv]: views of one projection (row stride in elements); decay fp32 [H].
-OME_API int ome_lightning_scan(const void* q, const void* k, const void* v, int64_t stride, const float* decay, float* state,
-                               void* out, const int* cu, const int* slot, const int* reset, int S, int H, int dk, int dv,
-                               int f32, hipStream_t stream) {
-  if (S <= 0) return 0;
-  if (bad_shape(H, H, dk, dv) || H > 65535) return -2;
-  const ScanArgs a{nullptr, nullptr, nullptr, stride, stride, nullptr, nullptr, 0, 0, decay, state, cu, slot, reset, H, H, dk, dv};
-  if (f32) return scan_by_width<float, LIGHTNING>(q, k, v, nullptr, nullptr, out, a, S, stream);
-  return scan_by_width<bf16, LIGHTNING>(q, k, v, nullptr, nullptr, out, a, S, stream);
+OME_API int ome_lightning_scan(const void* q, const void* k, const void* v, int64_t stride, const float* decay, float* ws,
+                               int chunks, float* state, void* out, const int* cu, const int* slot, const int* reset, int S,
+                               int H, int dk, int dv, int f32, hipStream_t stream) {
+  if (S <= 0 || chunks <= 0) return 0;
+  if (bad_shape(S, H, H, dk, dv)) return -2;
+  const PrepArgs p{stride, 0, 0, 1, nullptr, nullptr, decay, ws, cu, slot, reset, S, H, H, dk, dv};
+  const ScanArgs a{ws, stride, state, cu, slot, reset, H, dk, dv};
+  if (f32)
+    return chunked_by_width<float, LIGHTNING>(q, k, v, nullptr, nullptr, nullptr, nullptr, nullptr, p, a, out, chunks, false, stream);
+  return chunked_by_width<bf16, LIGHTNING>(q, k, v, nullptr, nullptr, nullptr, nullptr, nullptr, p, a, out, chunks, false, stream);
 }
 
 // The whole mixer core for sequences of one row each: z rows [decay inputs (H * dk) | output gate (H * dv)].
@@ -797,7 +883,7 @@ OME_API int ome_delta_step(const void* x, int64_t stride, const void* conv_w, vo
                            const void* norm_w, float eps, float* state, void* out, const int* cu, const int* slot,
                            const int* reset, int S, int H, int Hk, int dk, int dv, int f32, hipStream_t stream) {
   if (S <= 0) return 0;
-  if (bad_shape(H, Hk, dk, dv) || Hk > 65535 || K < 1 || K > 32) return -2;
+  if (bad_shape(S, H, Hk, dk, dv) || K < 1 || K > 32) return -2;
   const StepArgs a{stride, z_stride, b_stride, K, A_log, dt_bias, nullptr, eps, state, cu, slot, reset, H, Hk, dk, dv};
   if (f32) return step_by_width<float, DELTA>(x, nullptr, nullptr, conv_w, conv_state, z, b, norm_w, out, a, S, stream);
   return step_by_width<bf16, DELTA>(x, nullptr, nullptr, conv_w, conv_state, z, b, norm_w, out, a, S, stream);
@@ -807,7 +893,7 @@ OME_API int ome_lightning_step(const void* q, const void* k, const void* v, int6
                                float* state, void* out, const int* cu, const int* slot, const int* reset, int S, int H,
                                int dk, int dv, int f32, hipStream_t stream) {
   if (S <= 0) return 0;
-  if (bad_shape(H, H, dk, dv) || H > 65535) return -2;
+  if (bad_shape(S, H, H, dk, dv)) return -2;
   const StepArgs a{stride, 0, 0, 1, nullptr, nullptr, decay, 0.f, state, cu, slot, reset, H, H, dk, dv};
   if (f32) return step_by_width<float, LIGHTNING>(q, k, v, nullptr, nullptr, nullptr, nullptr, nullptr, out, a, S, stream);
   return step_by_width<bf16, LIGHTNING>(q, k, v, nullptr, nullptr, nullptr, nullptr, nullptr, out, a, S, stream);

@@ -1,5 +1,10 @@
 """Layer-list designs beside their closest existing model at equal size (``bench.py --arch-compare
-[--arch-design zavilorn|metitar|milenex|nivasun|pagatar]``).
+[--arch-design zavilorn|metitar|milenex|nivasun|pagatar|gisirax]``).
+
+Gisirax (gated delta rule with a decay per key channel, full causal attention beside lightning
+attention, tanh norms around every sublayer, group-routed SiLU-GLU experts, on a hashed token-pair
+embedding) stands beside a Qwen3-Next-style stack (gated delta rule with a decay per head, gated full
+attention, SiLU-GLU experts) of the same width, depth, layer order, head counts and expert sizes.
 
 Pagatar (chunked attention behind short convolutions with value mixing, minGRU, full latent attention,
 sigmoid-routed SiLU-GLU experts, output norms in channel groups and a learned average over depth)
@@ -164,6 +169,34 @@ def pagatar_config(s: dict, chunk: int = 1024) -> dict:
                      "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}}
     return {"architecture": "Pagatar", "layers": [att, gru, lat, att] * 2, "norm": {"eps": 1e-6, "groups": 4}, "vocab": s["vocab"],
             "width": s["width"], "max_positions": 8192}
+
+
+def gisirax_config(s: dict) -> dict:
+    """[channel delta x 3, attention || lightning] x 2 with 128-wide heads, as many key as value heads
+    in the delta rule, 4 taps, every layer with 32 experts in 8 groups, 4 groups kept, top 4."""
+    moe = {"kind": "moe", "expert": {"ff": s["eff"]},
+           "router": {"experts": s["experts"], "top": s["top"], "groups": {"count": 8, "keep": 4}, "scale": 2.0}}
+    H = s["heads"]
+    delta = {"type": "channel_delta", "mlp": moe, "mixer": {"heads": H, "kv_heads": H, "dim": 128, "vdim": 128, "conv": 4}}
+    par = {"type": "parallel", "mlp": moe,
+           "mixer": {"left": {"heads": H, "kv_heads": s["kv"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                              "rot": {"base": 500000.0, "dims": 128,
+                                      "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+                     "right": {"heads": H, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** -(1 + 7 * h / H) for h in range(H)]}}}
+    return {"architecture": "Gisirax", "layers": [delta, delta, delta, par] * 2, "norm": {"eps": 1e-6}, "vocab": s["vocab"],
+            "width": s["width"], "max_positions": 8192, "residual_mult": 0.5,
+            "embedding": {"scale": 1.0, "bigram": {"buckets": 65521, "mul_prev": 36313, "mul_cur": 27191}}}
+
+
+def qwen3_next_like_config(s: dict) -> dict:
+    """[gated delta net x 3, gated full attention] x 2 of the Gisirax stack's sizes, no shared expert."""
+    H = s["heads"]
+    return dict(architectures=["Qwen3NextForCausalLM"], model_type="qwen3_next", hidden_size=s["width"], num_hidden_layers=8,
+                num_attention_heads=H, num_key_value_heads=s["kv"], head_dim=128, intermediate_size=s["eff"],
+                moe_intermediate_size=s["eff"], num_experts=s["experts"], num_experts_per_tok=s["top"], norm_topk_prob=True,
+                linear_num_key_heads=H, linear_num_value_heads=H, linear_key_head_dim=128, linear_value_head_dim=128,
+                linear_conv_kernel_dim=4, full_attention_interval=4, partial_rotary_factor=1.0, rope_theta=500000.0,
+                vocab_size=s["vocab"], rms_norm_eps=1e-6, max_position_embeddings=8192, tie_word_embeddings=False)
 
 
 def gpt_oss_like_config(s: dict, window: int = 1024) -> dict:
@@ -859,8 +892,146 @@ def kernel_table_pagatar(T: int = 4096, B: int = 64, ctx: int = 4096, width: int
     return rows
 
 
+def kernel_table_gisirax(T: int = 4096, B: int = 64, ctx: int = 4096, width: int = 4096) -> list[dict]:
+    """Gisirax's kernels beside their like kernels (same columns as :func:`kernel_table`)."""
+    from ome_amd import ops
+    from ome_amd.models.config import plain_rope_table
+    from ome_amd.models.mixers import GroupRoutedMoE
+
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+
+    def pair(name, new, like, bytes_new, bytes_like, note="", iters=30):
+        tn, tl = _time_us(new, iters), _time_us(like, iters)
+        fn, fl = bytes_new / tn / 1e3 / HBM_GBS, bytes_like / tl / 1e3 / HBM_GBS
+        rows.append({"kernel": name, "us": round(tn, 1), "roofline": round(fn, 3), "like_us": round(tl, 1),
+                     "like_roofline": round(fl, 3), "vs_like": round(fl / max(fn, 1e-9), 2), "note": note})
+
+    def seqs(lens):
+        cu = torch.tensor([0] + torch.tensor(lens).cumsum(0).tolist(), dtype=torch.int32, device=dev)
+        n = len(lens)
+        return cu, torch.arange(n, dtype=torch.int32, device=dev), torch.zeros(n, dtype=torch.int32, device=dev)
+
+    torch.manual_seed(0)
+    H, d, Hq, Hkv, D, P = 32, 128, 32, 8, 128, 16
+    n = H * d
+    for R, tag, lens in ((T, "prefill, 2 sequences", [T // 2] * 2), (T, "prefill, 8 sequences", [T // 8] * 8),
+                         (T, "prefill, 1 sequence", [T]), (B, "decode", [1] * B)):
+        sq = seqs(lens)
+        S, single = len(lens), R == len(lens)
+        # ---- channel-decayed delta rule, conv to gated head output, vs conv + gated delta rule + gated head norm
+        p = torch.randn(R, 3 * n, device=dev).to(bf)
+        z = torch.randn(R, 2 * n, device=dev).to(bf)
+        ab = torch.randn(R, 2 * H, device=dev).to(bf)
+        cw = (torch.randn(3 * n, 4, device=dev) * 0.3).to(bf)
+        cs1 = torch.zeros(S, 3 * n, 3, device=dev, dtype=bf)
+        Al, dbc = torch.full((H,), -2.0, device=dev), torch.zeros(n, device=dev)
+        Al2, db = torch.zeros(H, device=dev), torch.zeros(H, device=dev)
+        gw = torch.ones(d, device=dev, dtype=bf)
+        st = torch.zeros(S, H, d, d, device=dev)
+
+        def like_delta():
+            c = ops.ssm_conv1d(p, cw, None, cs1, *sq)
+            o = ops.gdn_scan(c[:, :n], c[:, n:2 * n], c[:, 2 * n:], ab[:, :H], ab[:, H:], Al2, db, st, *sq, H, H)
+            return ops.gated_rmsnorm(o, z[:, :n], gw, d, 1e-6, norm_first=True, exact=True)
+
+        state_b, tail_b = S * H * d * d * 8, S * 3 * n * 3 * 4
+        pair(f"channel_delta 32 x 128 x 128 ({tag})",
+             lambda: ops.channel_delta(p, cw, cs1, z, ab[:, :H], Al, dbc, gw, 1e-6, st, sq, H, single_rows=single),
+             like_delta, state_b + tail_b + R * n * 12, state_b + tail_b + R * n * 10,
+             "convolution to gated head output; like: Qwen3-Next's convolution, scan and gated norm", 10)
+        # ---- lightning attention vs the gated delta rule scan of equal head shape
+        dec = torch.linspace(0.5, 0.99, H, device=dev)
+        pair(f"lightning_scan 32 x 128 x 128 ({tag})",
+             lambda: ops.lightning_scan(p[:, :n], p[:, n:2 * n], p[:, 2 * n:], dec, st, sq, single_rows=single),
+             lambda: ops.gdn_scan(p[:, :n], p[:, n:2 * n], p[:, 2 * n:], ab[:, :H], ab[:, H:], Al2, db, st, *sq, H, H),
+             state_b + R * n * 8, state_b + R * (n * 8 + 4 * H), "like: Qwen3-Next's gated delta rule", 10)
+    for R, tag in ((T, "prefill"), (B, "decode")):
+        # ---- tanh stream vs add + RMSNorm on a bf16 stream
+        x = torch.randn(R, width, device=dev)
+        y, y2 = (torch.randn(R, width, device=dev).to(bf) for _ in range(2))
+        w, b = torch.ones(width, device=dev, dtype=bf), torch.zeros(width, device=dev, dtype=bf)
+        rb, xb = x.to(bf), y.clone()
+        like = lambda: ops.fused_add_rmsnorm(xb, rb, w, 1e-6)   # noqa: E731
+        curve = (0.5, w, b)
+        pair(f"tanh_stream, one output ({tag})", lambda: ops.tanh_stream(x, curve, bf, post=curve, mult=0.3, y=y), like,
+             R * width * 12, R * width * 8, "fp32 stream: 12 B / element against 8; two curves")
+        pair(f"tanh_stream, two joined outputs ({tag})",
+             lambda: ops.tanh_stream(x, curve, bf, post=curve, mult=0.3, y=y, y2=y2, join=(w, w, 1e-6)), like, R * width * 14,
+             R * width * 8, "two RMS norms, then the curves")
+        # ---- norm over all heads + sigmoid gate vs the per-head norm + SiLU gate
+        o, g = torch.randn(R, n, device=dev).to(bf), torch.randn(R, n, device=dev).to(bf)
+        wn, gw = torch.ones(n, device=dev, dtype=bf), torch.ones(d, device=dev, dtype=bf)
+        head = lambda: ops.gated_rmsnorm(o, g, gw, d, 1e-6, norm_first=True)   # noqa: E731
+        pair(f"gated_rmsnorm over all heads, sigmoid ({tag})",
+             lambda: ops.gated_rmsnorm(o, g, wn, n, 1e-6, norm_first=True, exact=True, gate="sigmoid"), head, R * n * 6, R * n * 6,
+             "like: Qwen3-Next's norm per head")
+        # ---- attention input: rotation + cache write
+        n_pages = R // P + 2
+        kc = torch.zeros(n_pages, Hkv, P, D, device=dev, dtype=bf)
+        vc = torch.zeros(n_pages, Hkv, D, P, device=dev, dtype=bf)
+        C = (Hq + 2 * Hkv) * D
+        qkv = torch.randn(R, C, device=dev).to(bf)
+        pos = torch.arange(R, dtype=torch.int32, device=dev) % 2048
+        slots = torch.arange(R, dtype=torch.int32, device=dev) + P
+        cs = plain_rope_table(10000.0, 128, 2049, dev)
+        qo = torch.empty(R, Hq, D, device=dev, dtype=bf)
+        hn = torch.ones(D, device=dev, dtype=bf)
+        pair(f"wide_norm_rope_cache without norms, halves ({tag})",
+             lambda: ops.wide_norm_rope_cache(qkv[:, :Hq * D], qkv[:, Hq * D:(Hq + Hkv) * D], qkv[:, (Hq + Hkv) * D:], pos, cs, 128,
+                                              False, None, None, 0.0, qo, kc, vc, slots, Hq, Hkv, D, D),
+             lambda: ops.rope_qkv_cache(qkv, pos, cs, 128, qo, kc, vc, slots, Hq, Hkv, D, True, hn, hn, 1e-6), R * C * 4, R * C * 4)
+        # ---- routed feed-forward
+        E, k, ff = 32, 4, 2048
+        moe = GroupRoutedMoE(width, E, k, ff, 0.0, 8, 4, 0, 0.0, dev, bf, act=0, renorm=True, correction=False, scoring="sigmoid",
+                             group_score="top2", routed_scale=2.0)
+        moe.init_random(torch.Generator(device=dev).manual_seed(1), 0.02)
+        xx = torch.randn(R, width, device=dev).to(bf)
+        tw, tid = ops.moe_route(torch.randn(R, E, device=dev), k, True, "softmax")
+        touched = min(E, R * k) * 3 * ff * width * 2
+        pair(f"group-routed moe 32 experts in 8 groups top 4 ({tag})", lambda: moe.forward(xx),
+             lambda: ops.fused_moe(xx, tw, tid, moe.w13, moe.w2, 0, 1.0), touched, touched,
+             "new: router GEMM + route + grouped GEMMs + combine; like: grouped GEMMs + combine", 10)
+    # ---- full causal attention with one added to the denominator vs without
+    per = ctx // P
+    kc = (torch.randn(B * per + 1, Hkv, P, D, device=dev) * 0.3).to(bf)
+    vc = (torch.randn(B * per + 1, Hkv, D, P, device=dev) * 0.3).to(bf)
+    bt = (torch.arange(B * per, dtype=torch.int32, device=dev) + 1).view(B, per)
+    sl = torch.full((B,), ctx, dtype=torch.int32, device=dev)
+    q = (torch.randn(B, Hq, D, device=dev) * 0.3).to(bf)
+    ws = ops.DecodeWorkspace(B, Hq, D, ctx, 0, dev, parts=4)
+    sink = torch.zeros(Hq, device=dev)
+    kvb = B * Hkv * D * 2 * 2 * ctx
+    pair("attention decode 64 x 4096 ctx, plus one", lambda: ops.paged_decode(q, kc, vc, bt, sl, 0.09, ws, sinks=sink),
+         lambda: ops.paged_decode(q, kc, vc, bt, sl, 0.09, ws), kvb, kvb, "like: the plain softmax", 10)
+    q_lens = [2048, 2048]
+    Tq = sum(q_lens)
+    qp = (torch.randn(Tq, Hq, D, device=dev) * 0.3).to(bf)
+    cu = torch.tensor([0, 2048, 4096], dtype=torch.int32, device=dev)
+    kl = torch.tensor(q_lens, dtype=torch.int32, device=dev)
+    bt2 = (torch.arange(2 * 128, dtype=torch.int32, device=dev) + 1).view(2, 128)
+    items = torch.tensor(ops.prefill_work_items(q_lens, q_lens), dtype=torch.int32, device=dev)
+    fl = 4.0 * Hq * D * sum(i + 1 for i in range(2048)) * 2
+    tn = _time_us(lambda: ops.paged_prefill(qp, kc, vc, bt2, cu, kl, items, 0.09, sinks=sink), 10)
+    tl = _time_us(lambda: ops.paged_prefill(qp, kc, vc, bt2, cu, kl, items, 0.09), 10)
+    rows.append({"kernel": "attention prefill 2 x 2048 rows, plus one", "us": round(tn, 1), "roofline": round(fl / tn / 1e6 / 2.5e3, 3),
+                 "like_us": round(tl, 1), "like_roofline": round(fl / tl / 1e6 / 2.5e3, 3), "vs_like": round(tn / tl, 2),
+                 "note": "share of 2.5 PFLOP/s bf16; like: the plain softmax"})
+    return rows
+
+
 def run(sizes=("2k", "4k"), kernels: bool = True, only: str | None = None, design: str = "zavilorn") -> dict:
     out = {"throughput": [], "kernels": []}
+    if design == "gisirax":
+        for k in sizes:
+            s = X_SIZES[k]
+            if only in (None, "gisirax"):
+                out["throughput"].append(throughput(f"gisirax-{k}", gisirax_config(s)))
+            if only in (None, "qwen3-next"):
+                out["throughput"].append(throughput(f"qwen3-next-like-{k}", qwen3_next_like_config(s)))
+        if kernels:
+            out["kernels"] = kernel_table_gisirax()
+        return out
     if design == "pagatar":
         for k in sizes:
             s = X_SIZES[k]
@@ -918,10 +1089,11 @@ def main(argv=None) -> int:
     ap = argparse.ArgumentParser(description=__doc__)
     ap.add_argument("--sizes", default="2k,4k")
     ap.add_argument("--no-kernels", action="store_true")
-    ap.add_argument("--only", choices=["zavilorn", "nemotron", "metitar", "deepseek", "milenex", "gpt-oss", "nivasun", "pagatar"],
-                    default=None,
+    ap.add_argument("--only", choices=["zavilorn", "nemotron", "metitar", "deepseek", "milenex", "gpt-oss", "nivasun", "pagatar",
+                                       "gisirax", "qwen3-next"], default=None,
                     help="one stack (for kernel traces)")
-    ap.add_argument("--design", choices=["zavilorn", "metitar", "milenex", "nivasun", "pagatar"], default="zavilorn")
+    ap.add_argument("--design", choices=["zavilorn", "metitar", "milenex", "nivasun", "pagatar", "gisirax"],
+                    default="zavilorn")
     ap.add_argument("--no-throughput", action="store_true", help="the kernel table only")
     a = ap.parse_args(argv)
     res = run(() if a.no_throughput else tuple(a.sizes.split(",")), not a.no_kernels, a.only, a.design)

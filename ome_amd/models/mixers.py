@@ -317,11 +317,9 @@ class ChannelDeltaMixer(_Block):
     def forward(self, h: torch.Tensor, ctx: MixerCtx) -> torch.Tensor:
         p = linear(h, self.w_in)                                  # [T, q | k | v | a1 | g1 | b]
         z = linear(p[:, self.lr0:self.lr0 + self.lrw], self.w_lr)  # [T, decay | output gate]
-        single = ctx.meta.is_decode
-        rows = None if single else ctx.seq_rows(h)
         o = ops.channel_delta(p[:, :self.cd], self.conv_w, self.conv_state, z, p[:, self.b0:self.b0 + self.Hv], self.A_log,
-                              self.dt_bias, self.gnorm, self.eps, self.rec_state, ctx.seqs, self.Hk, rows=rows,
-                              single_rows=single)
+                              self.dt_bias, self.gnorm, self.eps, self.rec_state, ctx.seqs, self.Hk,
+                              single_rows=ctx.meta.is_decode)
         return linear(o, self.w_o)
 
 

@@ -2133,12 +2133,19 @@ def tanh_stream(x: torch.Tensor, pre: tuple, out_dtype, post: tuple | None = Non
     return out
 
 
-STATE_DIM_MAX = 512   # key channels per head of the matrix-state recurrences below
+STATE_DIM_MAX = 256   # key channels per head of the matrix-state recurrences below
+
+
+def _state_chunks(T: int, S: int, H: int, dk: int, delta: bool, device) -> tuple[torch.Tensor, int]:
+    """(workspace, chunk count) of a chunked scan over T rows of S sequences: chunks of 16 rows per
+    sequence, at most T / 16 full ones and S partial ones."""
+    chunks = (T + 15 * S) // 16
+    return torch.empty(chunks * H * load().ome_state_chunk_floats(dk, int(delta)), dtype=torch.float32, device=device), chunks
 
 
 def channel_delta(qkv: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor, z: torch.Tensor, b: torch.Tensor,
                   A_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor, eps: float, state: torch.Tensor,
-                  seqs: tuple, Hk: int, rows: tuple | None = None, single_rows: bool = False) -> torch.Tensor:
+                  seqs: tuple, Hk: int, single_rows: bool = False) -> torch.Tensor:
     """Core of a gated delta rule with one decay per head and key channel.  ``qkv`` rows [q (Hk*dk) | k
     (Hk*dk) | v (H*dv)] pass a causal depthwise convolution (``conv_w`` [C, K], tails ``conv_state``
     [slots, C, K-1]) + SiLU, q and k become unit vectors per head (q also / sqrt(dk)); ``z`` rows hold
@@ -2146,7 +2153,7 @@ def channel_delta(qkv: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Ten
     beta = sigmoid(``b`` [T, H]); per head S <- diag(g) S, u = beta (v - S^T k), S <- S + k u^T, o =
     S^T q (value head h reads key head h // (H / Hk)); returns o / rms(o) * ``norm_w`` * sigmoid(gate)
     as [T, H*dv].  ``state`` fp32 [slots, H, dv, dk] (S transposed).  ``seqs`` = (cu, slot, reset);
-    ``rows`` = :func:`seq_rows`; ``single_rows``: every sequence has one row (one launch)."""
+    ``single_rows``: every sequence has one row (one launch); otherwise chunks of 16 rows on fp32 MFMA."""
     cu, slot, reset = seqs
     H, dv, dk = state.shape[1:]
     T = qkv.shape[0]
@@ -2168,16 +2175,11 @@ def channel_delta(qkv: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Ten
              z.stride(0), b.data_ptr(), b.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), norm_w.data_ptr(), float(eps),
              state.data_ptr(), out.data_ptr(), *sp, H, Hk, dk, dv, f32, stream_ptr())
         return out
-    first, rslot = rows if rows is not None else seq_rows(seqs, T)
-    dkp = max(16, 1 << (dk - 1).bit_length())
-    ws = torch.empty(T * Hk * (2 * dkp + 1), dtype=torch.float32, device=qkv.device)
-    qn, kn, qk = ws[:T * Hk * dkp], ws[T * Hk * dkp:2 * T * Hk * dkp], ws[2 * T * Hk * dkp:]
+    ws, chunks = _state_chunks(T, slot.shape[0], H, dk, True, qkv.device)
     v = torch.empty(T, H * dv, dtype=qkv.dtype, device=qkv.device)
-    call("ome_delta_prep", qkv.data_ptr(), qkv.stride(0), conv_w.data_ptr(), conv_state.data_ptr(), K, _i32(first).data_ptr(),
-         _i32(rslot).data_ptr(), qn.data_ptr(), kn.data_ptr(), qk.data_ptr(), v.data_ptr(), T, H, Hk, dk, dv, f32, stream_ptr())
-    call("ome_delta_scan", qn.data_ptr(), kn.data_ptr(), qk.data_ptr(), v.data_ptr(), z.data_ptr(), z.stride(0), b.data_ptr(),
-         b.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(), out.data_ptr(), *sp, H, Hk, dk, dv, f32,
-         stream_ptr())
+    call("ome_delta_scan", qkv.data_ptr(), qkv.stride(0), conv_w.data_ptr(), conv_state.data_ptr(), K, z.data_ptr(), z.stride(0),
+         b.data_ptr(), b.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), v.data_ptr(), ws.data_ptr(), chunks, state.data_ptr(),
+         out.data_ptr(), *sp, H, Hk, dk, dv, f32, stream_ptr())
     if K > 1:
         call("ome_conv_tail", qkv.data_ptr(), qkv.stride(0), conv_state.data_ptr(), *sp, C, K, f32, stream_ptr())
     return gated_rmsnorm(out, z[:, H * dk:], norm_w, dv, eps, norm_first=True, exact=True, gate="sigmoid")
@@ -2199,9 +2201,15 @@ def lightning_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: tor
     assert q.shape[1] == k.shape[1] == H * dk and v.shape[1] == H * dv and dk <= STATE_DIM_MAX
     assert state.dtype == decay.dtype == torch.float32 and state.is_contiguous() and decay.numel() == H and decay.is_contiguous()
     sp = (_i32(cu).data_ptr(), _i32(slot).data_ptr(), _i32(reset).data_ptr(), slot.shape[0])
-    assert not single_rows or slot.shape[0] == T
-    call("ome_lightning_step" if single_rows else "ome_lightning_scan", q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0),
-         decay.data_ptr(), state.data_ptr(), out.data_ptr(), *sp, H, dk, dv, _f32(q, k, v), stream_ptr())
+    f32 = _f32(q, k, v)
+    if single_rows:
+        assert slot.shape[0] == T
+        call("ome_lightning_step", q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), decay.data_ptr(), state.data_ptr(),
+             out.data_ptr(), *sp, H, dk, dv, f32, stream_ptr())
+        return out
+    ws, chunks = _state_chunks(T, slot.shape[0], H, dk, False, q.device)
+    call("ome_lightning_scan", q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), decay.data_ptr(), ws.data_ptr(), chunks,
+         state.data_ptr(), out.data_ptr(), *sp, H, dk, dv, f32, stream_ptr())
     return out
 
 

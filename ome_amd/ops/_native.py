@@ -49,10 +49,11 @@ _SIGNATURES = {
                             i32, vp],
         "ome_tanh_stream": [vp, i64, vp, i64, vp, i64, vp, vp, f32, f32, f32, vp, vp, f32, vp, vp, vp, i64, i32, i32, i32,
                             vp],
-        "ome_delta_prep": [vp, i64, vp, vp, i32, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp],
         "ome_conv_tail": [vp, i64, vp, vp, vp, vp, i32, i32, i32, i32, vp],
-        "ome_delta_scan": [vp, vp, vp, vp, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp],
-        "ome_lightning_scan": [vp, vp, vp, i64, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp],
+        "ome_state_chunk_floats": [i32, i32],
+        "ome_delta_scan": [vp, i64, vp, vp, i32, vp, i64, vp, i64, vp, vp, vp, vp, i32, vp, vp, vp, vp, vp, i32, i32, i32,
+                           i32, i32, i32, vp],
+        "ome_lightning_scan": [vp, vp, vp, i64, vp, vp, i32, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp],
         "ome_delta_step": [vp, i64, vp, vp, i32, vp, i64, vp, i64, vp, vp, vp, f32, vp, vp, vp, vp, vp, i32, i32, i32, i32,
                            i32, i32, vp],
         "ome_lightning_step": [vp, vp, vp, i64, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp],
