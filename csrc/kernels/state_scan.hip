@@ -33,9 +33,17 @@ template <typename T>
 __device__ __forceinline__ float silu(float x) {
   return x * sigm<T>(x);
 }
-__device__ __forceinline__ float softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+// (16-bit models: the hardware's log of 1 + e^-|x|, absolute error of an fp32 rounding of 1)
+template <typename T>
+__device__ __forceinline__ float softplus(float x) {
+  if constexpr (sizeof(T) == 4) return x > 20.f ? x : log1pf(expf(x));
+  else return fmaxf(x, 0.f) + __logf(1.f + __expf(-fabsf(x)));
+}
 // decay factor of a raw decay input (A = exp(A_log) of the head)
-__device__ __forceinline__ float decay_of(float z, float bias, float A) { return expf(-A * softplus(z + bias)); }
+template <typename T>
+__device__ __forceinline__ float decay_of(float z, float bias, float A) {
+  return ex<T>(-A * softplus<T>(z + bias));
+}
 
 // sum over aligned groups of L lanes, result in all of them
 template <int L>
@@ -107,6 +115,10 @@ __device__ __forceinline__ int chunks_before(const int* __restrict__ cu, int s) 
 
 enum { DELTA = 0, LIGHTNING = 1 };
 
+__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
 // What `chunk_prep` leaves for `chunk_scan`, per (chunk, head), in floats: the operands of the state
 // products [CH][DKP] each (delta only: -G k), G q, the write keys transposed [DKP][CH], the state's decay over
 // the chunk [DKP], the CH x CH matrices (delta only: the solved write matrix), the read-out of the writes.
@@ -120,7 +132,7 @@ struct PrepArgs {
   int64_t stride, z_stride, b_stride;   // rows of the projection (q, k, v / lightning: q, k), z, b
   int K;                                // taps
   const float *A_log, *dt_bias, *decay;
-  float* ws;                            // [chunks][H] chunk operands
+  float* ws;                            // [H][chunks] chunk operands
   const int *cu, *slot, *reset;
   int S, H, Hk, dk, dv;
 };
@@ -138,10 +150,18 @@ __device__ __forceinline__ void conv_rows(const T* __restrict__ x, int64_t strid
       const int rr = min(max(r - (KT - 1) + i, r0), last);
       ldn<T, N, VEC>(x + (int64_t)rr * stride + ch, xs[i]);
     }
+    constexpr int W = N * KT;          // neighbouring taps of the lane's channels
+    float wf[W];
+    if constexpr (VEC && (W == 4 || W == 8)) {
+      ldn<T, W, true>(w + (int64_t)ch * KT, wf);
+    } else {
+#pragma unroll
+      for (int i = 0; i < W; ++i) wf[i] = (float)w[(int64_t)ch * KT + i];
+    }
 #pragma unroll
     for (int n = 0; n < N; ++n)
 #pragma unroll
-      for (int j = 0; j < KT; ++j) wt[j][n] = (float)w[(int64_t)(ch + n) * KT + j];
+      for (int j = 0; j < KT; ++j) wt[j][n] = wf[n * KT + j];
     if (r - r0 < KT - 1) {      // rows before the step come from the tail
 #pragma unroll
       for (int i = 0; i < KT - 1; ++i) {
@@ -182,8 +202,7 @@ __device__ __forceinline__ void conv_rows(const T* __restrict__ x, int64_t strid
 // One workgroup per (chunk, head).  N channels of q / k per lane (64 N >= DKP), four rows per wave.
 //   delta      A_ts = beta_t sum_c k_t k_s G_t / G_s (s < t);  the chunk's writes solve (1 + A) u = beta (v - (G k) S)
 //   both       B_ts = sum_c q_t k_s G_t / G_s (s <= t):        o = (G q) S + B u
-// with G_t the product of the decays from the chunk's start (ratios are powers of two of differences, which
-// never grow).  Rows beyond the sequence are empty: no key, no decay, nothing written.
+// with G_t the product of the decays from the chunk's start.  Rows beyond the sequence are empty: no key, no decay, nothing written.
 template <typename T, int DKP, int MODE, int KT, bool VEC>
 __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x, const T* __restrict__ k_in,
                                                          const T* __restrict__ w, const T* __restrict__ conv_state,
@@ -193,7 +212,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
   typedef ChunkLayout<DKP, MODE> Lay;
   __shared__ __attribute__((aligned(16))) float sq[CH][LD], sk[CH][LD], sa[MODE == DELTA ? CH : 1][LD];
   __shared__ __attribute__((aligned(16))) float sA[CH][CH + 4];
-  __shared__ float sb[CH + 1];
+  __shared__ float sb[CH + 1], part[2][4][CH * CH];
   int s = 0, c = 0;
   if (!find_chunk(a.cu, a.S, blockIdx.x, s, c)) return;   // uniform per block
   const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
@@ -201,8 +220,19 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
   const int r0 = a.cu[s], r1 = a.cu[s + 1], ra = r0 + c * CH, nr = min(CH, r1 - ra), last = r1 - 1;
   const int64_t slot = a.slot[s];
   const bool fresh = a.reset[s] != 0;
-  float* ws = a.ws + ((int64_t)blockIdx.x * a.H + h) * Lay::SIZE;
+  float* ws = a.ws + ((int64_t)h * gridDim.x + blockIdx.x) * Lay::SIZE;
   const int ch0 = lane * N, row0 = wv * RW;
+  constexpr int NZ = CH * DKP / 256;      // decays per thread, all of one channel
+  T zr[NZ], br = (T)0.f;
+  float dtb = 0.f;
+  if constexpr (MODE == DELTA) {          // (requested first, needed last)
+    const int cc = min(tid % DKP, dk - 1);
+    dtb = a.dt_bias[(int64_t)h * dk + cc];
+#pragma unroll
+    for (int u = 0; u < NZ; ++u)
+      zr[u] = z[(int64_t)min(ra + (tid + 256 * u) / DKP, last) * a.z_stride + (int64_t)h * dk + cc];
+    br = b[(int64_t)min(ra + tid % CH, last) * a.b_stride + h];
+  }
 
   // ---- queries and keys of the wave's rows into LDS
   float q[RW][N], k[RW][N];
@@ -241,7 +271,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
         ssq += q[i][n] * q[i][n];
         ssk += k[i][n] * k[i][n];
       }
-      const float iq = rd / sqrtf(wave_sum(ssq) + 1e-6f), ik = 1.f / sqrtf(wave_sum(ssk) + 1e-6f);
+      const float iq = rd / sqrtf(lanes_sum<64>(ssq) + 1e-6f), ik = 1.f / sqrtf(lanes_sum<64>(ssk) + 1e-6f);
 #pragma unroll
       for (int n = 0; n < N; ++n) {
         q[i][n] *= iq;
@@ -271,14 +301,6 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
 
   // ---- decays (log2), write strengths, values
   if constexpr (MODE == DELTA) {
-    const float A = expf(a.A_log[h]) * 1.44269504088896341f;
-    for (int e = tid; e < CH * DKP; e += 256) {
-      const int t = e / DKP, cc = e % DKP;
-      sa[t][cc] = t < nr && cc < dk
-                      ? -A * softplus((float)z[(int64_t)(ra + t) * a.z_stride + (int64_t)h * dk + cc] + a.dt_bias[(int64_t)h * dk + cc])
-                      : 0.f;
-    }
-    if (tid < CH) sb[tid] = tid < nr ? sigm<float>((float)b[(int64_t)(ra + tid) * a.b_stride + h]) : 0.f;
     constexpr int NV = VEC ? 2 : 1;
     const int C = 2 * kd + a.H * dv;
     for (int cv = lane * NV; cv < dv && row0 < nr; cv += 64 * NV) {
@@ -294,6 +316,13 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
           for (int n = 0; n < NV; ++n) vo[n] = (T)t[i][n];
         }
     }
+    const float A = expf(a.A_log[h]) * 1.44269504088896341f;
+#pragma unroll
+    for (int u = 0; u < NZ; ++u) {
+      const int t = (tid + 256 * u) / DKP, cc = tid % DKP;
+      sa[t][cc] = t < nr && cc < dk ? -A * softplus<T>((float)zr[u] + dtb) : 0.f;
+    }
+    if (tid < CH) sb[tid] = tid < nr ? sigm<float>((float)br) : 0.f;
     __syncthreads();
     for (int cc = tid; cc < DKP; cc += 256) {   // running sums over the chunk
       float acc = 0.f;
@@ -308,35 +337,62 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
   }
   __syncthreads();
 
-  // ---- the CH x CH products, one pair of rows per thread
+  // ---- the CH x CH products (on fp32 MFMA: K order permuted as in the scan, the waves split the channels)
+  float kk = 0.f, qk = 0.f;
+  const int pt = tid / CH, pu = tid % CH;     // this thread's pair of rows
   {
-    const int t = tid / CH, u = tid % CH;
-    float kk = 0.f, qk = 0.f;
-#pragma unroll 4
-    for (int cc = 0; cc < DKP; cc += 4) {
-      const f32x4 ku = *reinterpret_cast<const f32x4*>(&sk[u][cc]), qt = *reinterpret_cast<const f32x4*>(&sq[t][cc]);
-      if constexpr (MODE == DELTA) {
-        const f32x4 kt = *reinterpret_cast<const f32x4*>(&sk[t][cc]);
-        const f32x4 at = *reinterpret_cast<const f32x4*>(&sa[t][cc]), au = *reinterpret_cast<const f32x4*>(&sa[u][cc]);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const float f = ku[e] * __builtin_amdgcn_exp2f(fminf(at[e] - au[e], 0.f));   // (pairs u > t are dropped below)
-          kk += kt[e] * f;
-          qk += qt[e] * f;
-        }
-      } else {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) qk += qt[e] * ku[e];
-      }
-    }
+    constexpr int M = DKP / 16;
+    const int g = lane >> 4, li = lane & 15;
+    bool wide = false;      // decays of the chunk beyond what the factored form can hold
     if constexpr (MODE == DELTA) {
-      sA[t][u] = u < t ? sb[t] * kk : 0.f;
-      ws[Lay::BM + tid] = u <= t ? qk : 0.f;
-    } else {
-      ws[Lay::BM + tid] = u <= t ? qk * sb[t - u] : 0.f;
+      for (int cc = lane; cc < DKP; cc += 64) wide |= sa[CH - 1][cc] < -110.f;
+      wide = __ballot(wide) != 0;      // (every wave looks at all channels: uniform over the block)
+    }
+    if (!wide) {
+      // G_t / G_u = 2^(a_t - a_mid) 2^(a_mid - a_u): either factor at most 2^110
+      f32x4 ckk = f32x4{0.f, 0.f, 0.f, 0.f}, cqk = ckk;
+      for (int m = wv; m < M; m += 4) {
+        const int cc = 16 * m + 4 * g;
+        const f32x4 kr = *reinterpret_cast<const f32x4*>(&sk[li][cc]);
+        f32x4 ka = kr, kb = kr, qa = *reinterpret_cast<const f32x4*>(&sq[li][cc]);
+        if constexpr (MODE == DELTA) {
+          const f32x4 al = *reinterpret_cast<const f32x4*>(&sa[li][cc]), am = *reinterpret_cast<const f32x4*>(&sa[CH / 2 - 1][cc]);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const float f = __builtin_amdgcn_exp2f(al[r] - am[r]);
+            ka[r] *= f;
+            qa[r] *= f;
+            kb[r] *= __builtin_amdgcn_exp2f(am[r] - al[r]);
+          }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          if constexpr (MODE == DELTA) ckk = mfma4(ka[r], kb[r], ckk);
+          cqk = mfma4(qa[r], kb[r], cqk);
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        if constexpr (MODE == DELTA) part[0][wv][(4 * g + r) * CH + li] = ckk[r];
+        part[1][wv][(4 * g + r) * CH + li] = cqk[r];
+      }
+      __syncthreads();
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        if constexpr (MODE == DELTA) kk += part[0][u][tid];
+        qk += part[1][u][tid];
+      }
+    } else if constexpr (MODE == DELTA) {     // one pair of rows per thread, every ratio on its own
+      for (int cc = 0; cc < DKP; ++cc) {
+        const float f = sk[pu][cc] * __builtin_amdgcn_exp2f(fminf(sa[pt][cc] - sa[pu][cc], 0.f));
+        kk += sk[pt][cc] * f;
+        qk += sq[pt][cc] * f;
+      }
     }
   }
   if constexpr (MODE == DELTA) {
+    sA[pt][pu] = pu < pt ? sb[pt] * kk : 0.f;
+    ws[Lay::BM + tid] = pu <= pt ? qk : 0.f;
     __syncthreads();
     if (wv == 0) {   // X = (1 + A)^-1 column by column; the write matrix is X diag(beta)
       float X[CH];
@@ -351,18 +407,35 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(const T* __restrict__ x
 #pragma unroll
         for (int t = 0; t < CH; ++t) ws[Lay::TB + t * CH + lane] = X[t] * sb[lane];
     }
+  } else {
+    ws[Lay::BM + tid] = pu <= pt ? qk * sb[pt - pu] : 0.f;
   }
   // ---- operands of the state products
-  for (int e = tid; e < CH * DKP; e += 256) {
+  for (int e = 4 * tid; e < CH * DKP; e += 1024) {
     const int t = e / DKP, cc = e % DKP;
-    const float g = MODE == DELTA ? __builtin_amdgcn_exp2f(sa[t][cc]) : sb[min(t + 1, nr)];
-    if constexpr (MODE == DELTA) ws[Lay::GK + e] = -g * sk[t][cc];
-    ws[Lay::GQ + e] = g * sq[t][cc];
+    f32x4 gq = *reinterpret_cast<const f32x4*>(&sq[t][cc]);
+    if constexpr (MODE == DELTA) {
+      f32x4 gk = *reinterpret_cast<const f32x4*>(&sk[t][cc]);
+      const f32x4 al = *reinterpret_cast<const f32x4*>(&sa[t][cc]);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float f = __builtin_amdgcn_exp2f(al[r]);
+        gq[r] *= f;
+        gk[r] *= -f;
+      }
+      *reinterpret_cast<f32x4*>(ws + Lay::GK + e) = gk;
+    } else {
+      gq *= sb[min(t + 1, nr)];
+    }
+    *reinterpret_cast<f32x4*>(ws + Lay::GQ + e) = gq;
   }
-  for (int e = tid; e < CH * DKP; e += 256) {
+  for (int e = 4 * tid; e < CH * DKP; e += 1024) {
     const int cc = e / CH, t = e % CH;
-    const float g = MODE == DELTA ? __builtin_amdgcn_exp2f(sa[CH - 1][cc] - sa[t][cc]) : sb[max(nr - 1 - t, 0)];
-    ws[Lay::KT + e] = g * sk[t][cc];
+    f32x4 kt;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      kt[r] = sk[t + r][cc] * (MODE == DELTA ? __builtin_amdgcn_exp2f(sa[CH - 1][cc] - sa[t + r][cc]) : sb[max(nr - 1 - t - r, 0)]);
+    *reinterpret_cast<f32x4*>(ws + Lay::KT + e) = kt;
   }
   for (int cc = tid; cc < DKP; cc += 256) ws[Lay::GC + cc] = MODE == DELTA ? __builtin_amdgcn_exp2f(sa[CH - 1][cc]) : sb[nr];
 }
@@ -386,27 +459,24 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ x,
 
 struct ScanArgs {
   const float* ws;
+  int chunks;
   int64_t v_stride;
   float* state;
   const int *cu, *slot, *reset;
   int H, dk, dv;
 };
 
-__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
-}
-
 // Walks the chunks of one (sequence, head); wave w owns 16 value columns.  Accumulator layout of the
 // 16 x 16 x 4 product: lane (g = lane / 16, li = lane % 16) holds rows 4 g + r of column li; as the second
 // operand lane (g, li) supplies row g.  The order of a dot product's terms is free, so product r of a tile takes
 // the rows {4 g + r}: an accumulator's element r IS the second operand, and the first operand's four elements
 // are neighbours in LDS.  The state (channels 16 m + 4 g + r of column li) never leaves its accumulators.
-template <typename T, int DKP, int MODE, int NBUF>
-__global__ __launch_bounds__(256) void chunk_scan_kernel(const T* __restrict__ v, T* __restrict__ out, ScanArgs a) {
+template <typename T, int DKP, int MODE>
+__global__ __launch_bounds__(256, 2) void chunk_scan_kernel(const T* __restrict__ v, T* __restrict__ out, ScanArgs a) {
   typedef ChunkLayout<DKP, MODE> Lay;
   constexpr int M = DKP / 16, LD = DKP + 4, LT = CH + 4;
   constexpr int OGK = 0, OGQ = MODE == DELTA ? CH * LD : 0, OKT = OGQ + CH * LD, OGC = OKT + DKP * LT, OTB = OGC + DKP,
-                OBM = OTB + (MODE == DELTA ? CH * LT : 0), OSZ = OBM + CH * LT;   // the same operands with padded rows
+                OBM = OTB + (MODE == DELTA ? CH * LT : 0), OSZ = OBM + CH * LT + 4;   // the same operands with padded rows
   constexpr int NF = (Lay::SIZE / 4 + 255) / 256;   // 16-byte loads per thread and chunk
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, g = lane >> 4, li = lane & 15;
@@ -430,58 +500,72 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(const T* __restrict__ v
     }
   }
   const int nc = (r1 - r0 + CH - 1) / CH;
-  const float* ws = a.ws + ((int64_t)chunks_before(a.cu, s) * a.H + h) * Lay::SIZE;
-  f32x4 pre[NF], pv;
-  auto fetch = [&](int c) {
-    const f32x4* p = reinterpret_cast<const f32x4*>(ws + (int64_t)c * a.H * Lay::SIZE);
+  const float* ws = a.ws + ((int64_t)h * a.chunks + chunks_before(a.cu, s)) * Lay::SIZE;
+  // operands and values of the next chunk in flight (values unconverted: a use would wait for the load)
+  f32x4 pre[NF];
+  T pv[4];
+  const T* vp = v + (int64_t)h * dv + (on ? col : 0);
+  int at[NF];          // where they go in LDS (the surplus of the last round: four unused floats)
+#pragma unroll
+  for (int u = 0; u < NF; ++u) {
+    const int e = 4 * (tid + 256 * u);
+    if (e >= Lay::SIZE) at[u] = OSZ - 4;
+    else if (MODE == DELTA && e < Lay::GQ) at[u] = OGK + e / DKP * LD + e % DKP;
+    else if (e < Lay::KT) at[u] = OGQ + (e - Lay::GQ) / DKP * LD + (e - Lay::GQ) % DKP;
+    else if (e < Lay::GC) at[u] = OKT + (e - Lay::KT) / CH * LT + (e - Lay::KT) % CH;
+    else if (e < Lay::TB) at[u] = OGC + e - Lay::GC;
+    else if (e < Lay::BM) at[u] = OTB + (e - Lay::TB) / CH * LT + (e - Lay::TB) % CH;
+    else at[u] = OBM + (e - Lay::BM) / CH * LT + (e - Lay::BM) % CH;
+  }
+  // loads i0 .. i1 - 1 of the NF + 4 of chunk c (beyond the sequence: its last chunk again)
+  auto fetch_part = [&](int c, int i0, int i1) {
+    c = min(c, nc - 1);
+    const f32x4* p = reinterpret_cast<const f32x4*>(ws + (int64_t)c * Lay::SIZE);
 #pragma unroll
     for (int u = 0; u < NF; ++u)
-      if (tid + 256 * u < Lay::SIZE / 4) pre[u] = p[tid + 256 * u];
+      if (u >= i0 && u < i1) pre[u] = p[min(tid + 256 * u, Lay::SIZE / 4 - 1)];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int row = r0 + c * CH + 4 * g + r;
-      float t = 0.f;
-      if (on && row < r1) {
-        t = (float)v[(int64_t)row * a.v_stride + (int64_t)h * dv + col];
-        if constexpr (MODE == LIGHTNING) t = silu<T>(t);
-      }
-      pv[r] = t;
-    }
+    for (int r = 0; r < 4; ++r)
+      if (NF + r >= i0 && NF + r < i1) pv[r] = vp[(int64_t)min(r0 + c * CH + 4 * g + r, r1 - 1) * a.v_stride];
   };
   auto store = [&](float* p) {
 #pragma unroll
-    for (int u = 0; u < NF; ++u) {
-      const int e = 4 * (tid + 256 * u);
-      if (e >= Lay::SIZE) continue;
-      int o;
-      if (MODE == DELTA && e < Lay::GQ) o = OGK + e / DKP * LD + e % DKP;
-      else if (e < Lay::KT) o = OGQ + (e - Lay::GQ) / DKP * LD + (e - Lay::GQ) % DKP;
-      else if (e < Lay::GC) o = OKT + (e - Lay::KT) / CH * LT + (e - Lay::KT) % CH;
-      else if (e < Lay::TB) o = OGC + e - Lay::GC;
-      else if (e < Lay::BM) o = OTB + (e - Lay::TB) / CH * LT + (e - Lay::TB) % CH;
-      else o = OBM + (e - Lay::BM) / CH * LT + (e - Lay::BM) % CH;
-      *reinterpret_cast<f32x4*>(p + o) = pre[u];
-    }
+    for (int u = 0; u < NF; ++u) *reinterpret_cast<f32x4*>(p + at[u]) = pre[u];
   };
   auto rd4 = [](const float* p) { return *reinterpret_cast<const f32x4*>(p); };
-  fetch(0);
-  int buf = 0;
+  auto values = [&](int c) {
+    f32x4 R;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float t = MODE == LIGHTNING ? silu<T>((float)pv[r]) : (float)pv[r];
+      R[r] = r0 + c * CH + 4 * g + r < r1 ? t : 0.f;
+    }
+    return R;
+  };
+  fetch_part(0, 0, NF + 4);
+  store(sm);
+  f32x4 R = values(0);
+  fetch_part(1, 0, NF + 4);
+  __syncthreads();
   for (int c = 0; c < nc; ++c) {
-    float* p = sm + buf * OSZ;
-    if (NBUF == 1 && c > 0) __syncthreads();   // the previous chunk's readers
-    store(p);
-    f32x4 R = pv, O = f32x4{0.f, 0.f, 0.f, 0.f};
-    __syncthreads();    // (two buffers: the one written next was last read before this barrier)
-    if (c + 1 < nc) fetch(c + 1);
+    const float* p = sm + (c & 1) * OSZ;
+    f32x4 O = f32x4{0.f, 0.f, 0.f, 0.f}, Vn = O;
     if constexpr (MODE == DELTA) {
+      f32x4 gk[2], gq[2];      // (the next tile's operands are read while this one's products run)
+      gk[0] = rd4(p + OGK + li * LD + 4 * g);
+      gq[0] = rd4(p + OGQ + li * LD + 4 * g);
 #pragma unroll
       for (int m = 0; m < M; ++m) {
-        const f32x4 gk = rd4(p + OGK + li * LD + 16 * m + 4 * g), gq = rd4(p + OGQ + li * LD + 16 * m + 4 * g);
+        if (m + 1 < M) {
+          gk[(m + 1) & 1] = rd4(p + OGK + li * LD + 16 * (m + 1) + 4 * g);
+          gq[(m + 1) & 1] = rd4(p + OGQ + li * LD + 16 * (m + 1) + 4 * g);
+        }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          R = mfma4(gk[r], S[m][r], R);
-          O = mfma4(gq[r], S[m][r], O);
+          R = mfma4(gk[m & 1][r], S[m][r], R);
+          O = mfma4(gq[m & 1][r], S[m][r], O);
         }
+        __builtin_amdgcn_sched_barrier(0);
       }
       const f32x4 tb = rd4(p + OTB + li * LT + 4 * g);
       f32x4 U = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -490,30 +574,45 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(const T* __restrict__ v
       R = U;
     } else {
       f32x4 O2 = f32x4{0.f, 0.f, 0.f, 0.f};
+      f32x4 gq[M];
 #pragma unroll
-      for (int m = 0; m < M; ++m) {
-        const f32x4 gq = rd4(p + OGQ + li * LD + 16 * m + 4 * g);
+      for (int m = 0; m < M; ++m) gq[m] = rd4(p + OGQ + li * LD + 16 * m + 4 * g);
+#pragma unroll
+      for (int m = 0; m < M; ++m)
 #pragma unroll
         for (int r = 0; r < 4; r += 2) {
-          O = mfma4(gq[r], S[m][r], O);
-          O2 = mfma4(gq[r + 1], S[m][r + 1], O2);
+          O = mfma4(gq[m][r], S[m][r], O);
+          O2 = mfma4(gq[m][r + 1], S[m][r + 1], O2);
         }
-      }
       O += O2;
     }
-#pragma unroll
-    for (int m = 0; m < M; ++m) S[m] *= rd4(p + OGC + 16 * m + 4 * g);
+    if (c + 1 < nc) {      // the other buffer was last read before the barrier; a whole chunk's time for the next loads
+      store(sm + ((c + 1) & 1) * OSZ);
+      Vn = values(c + 1);
+    }
     const f32x4 bm = rd4(p + OBM + li * LT + 4 * g);
+    f32x4 kt[M], gc[M];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) O = mfma4(bm[r], R[r], O);
+    for (int m = 0; m < M; ++m) {
+      gc[m] = rd4(p + OGC + 16 * m + 4 * g);
+      kt[m] = rd4(p + OKT + (16 * m + li) * LT + 4 * g);
+    }
 #pragma unroll
-    for (int m = 0; m < M; m += 2) {
-      const f32x4 k0 = rd4(p + OKT + (16 * m + li) * LT + 4 * g);
-      const f32x4 k1 = M > 1 ? rd4(p + OKT + (16 * (m + (M > 1)) + li) * LT + 4 * g) : k0;
+    for (int m = 0; m < M; ++m) S[m] *= gc[m];
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        S[m] = mfma4(k0[r], R[r], S[m]);
-        if constexpr (M > 1) S[m + 1] = mfma4(k1[r], R[r], S[m + 1]);
+    for (int r = 0; r < 4; ++r) {     // the loads of the chunk after next go out between the products
+      O = mfma4(bm[r], R[r], O);
+#pragma unroll
+      for (int m = 0; m < M; ++m) {
+        S[m] = mfma4(kt[m][r], R[r], S[m]);
+        constexpr int STEP = 4 * M / (NF + 4) > 0 ? 4 * M / (NF + 4) : 1;
+        if ((r * M + m) % STEP == STEP - 1 || r * M + m == 4 * M - 1) {
+          const int i = (r * M + m) / STEP;
+          if (r * M + m < 4 * M - 1) fetch_part(c + 2, i, i + 1);
+          else fetch_part(c + 2, i, NF + 4);
+          __builtin_amdgcn_sched_barrier(0);
+        }
       }
     }
 #pragma unroll
@@ -521,7 +620,8 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(const T* __restrict__ v
       const int row = r0 + c * CH + 4 * g + r;
       if (on && row < r1) out[((int64_t)row * a.H + h) * dv + col] = (T)O[r];
     }
-    if constexpr (NBUF == 2) buf ^= 1;
+    R = Vn;
+    __syncthreads();
   }
   if (!on) return;
 #pragma unroll
@@ -656,7 +756,7 @@ __global__ __launch_bounds__(256) void state_step_kernel(const T* __restrict__ q
         for (int u = 0; u < NU; ++u) {
           const int c = lane + 64 * u;
           if (c < DKP)
-            sg[c] = c < dk ? decay_of((float)z[(int64_t)row * a.z_stride + (int64_t)h * dk + c], a.dt_bias[(int64_t)h * dk + c], A)
+            sg[c] = c < dk ? decay_of<T>((float)z[(int64_t)row * a.z_stride + (int64_t)h * dk + c], a.dt_bias[(int64_t)h * dk + c], A)
                            : 0.f;
         }
       }
@@ -776,11 +876,20 @@ int chunked(const void* x, const void* k, const void* v_in, const void* w, const
   }
 #undef PREP
   OME_CHECK_LAUNCH();
-  constexpr int LD = DKP + 4, LT = CH + 4, NBUF = DKP <= 128 ? 2 : 1;
-  constexpr int lds = NBUF * ((MODE == DELTA ? 2 : 1) * CH * LD + DKP * LT + DKP + (MODE == DELTA ? 2 : 1) * CH * LT) * 4;
-  static_assert(lds <= 64 * 1024 && Lay::SIZE % 4 == 0, "chunk operands in LDS");
+  constexpr int LD = DKP + 4, LT = CH + 4;
+  constexpr int lds = 2 * ((MODE == DELTA ? 2 : 1) * CH * LD + DKP * LT + DKP + (MODE == DELTA ? 2 : 1) * CH * LT + 4) * 4;
+  static_assert(lds <= 160 * 1024 && Lay::SIZE % 4 == 0, "chunk operands in LDS");
+  if constexpr (lds > 64 * 1024) {
+    static bool done = false;   // (per instantiation; repeating the call is harmless)
+    if (!done) {
+      const hipError_t e = hipFuncSetAttribute((const void*)chunk_scan_kernel<T, DKP, MODE>,
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+      if (e != hipSuccess) return (int)e;
+      done = true;
+    }
+  }
   const dim3 sg(p.S, p.H, (p.dv + 63) / 64);
-  chunk_scan_kernel<T, DKP, MODE, NBUF><<<sg, 256, lds, stream>>>((const T*)v_in, (T*)out, a);
+  chunk_scan_kernel<T, DKP, MODE><<<sg, 256, lds, stream>>>((const T*)v_in, (T*)out, a);
   OME_CHECK_LAUNCH();
   return 0;
 }
@@ -857,7 +966,7 @@ OME_API int ome_delta_scan(const void* x, int64_t stride, const void* conv_w, co
   if (S <= 0 || chunks <= 0) return 0;
   if (bad_shape(S, H, Hk, dk, dv) || K < 1 || K > 32) return -2;
   const PrepArgs p{stride, z_stride, b_stride, K, A_log, dt_bias, nullptr, ws, cu, slot, reset, S, H, Hk, dk, dv};
-  const ScanArgs a{ws, (int64_t)H * dv, state, cu, slot, reset, H, dk, dv};
+  const ScanArgs a{ws, chunks, (int64_t)H * dv, state, cu, slot, reset, H, dk, dv};
   const int N = padded_dk(dk) > 64 ? padded_dk(dk) / 64 : 1, A = N > 2 ? N : 2;   // elements a vector access needs aligned
   const bool vec = N > 1 && dk % A == 0 && dv % 2 == 0 && stride % A == 0 && ((uintptr_t)x & (A * (f32 ? 4 : 2) - 1)) == 0;
   if (f32) return chunked_by_width<float, DELTA>(x, nullptr, v, conv_w, conv_state, z, b, v, p, a, out, chunks, vec, stream);
@@ -871,7 +980,7 @@ OME_API int ome_lightning_scan(const void* q, const void* k, const void* v, int6
   if (S <= 0 || chunks <= 0) return 0;
   if (bad_shape(S, H, H, dk, dv)) return -2;
   const PrepArgs p{stride, 0, 0, 1, nullptr, nullptr, decay, ws, cu, slot, reset, S, H, H, dk, dv};
-  const ScanArgs a{ws, stride, state, cu, slot, reset, H, dk, dv};
+  const ScanArgs a{ws, chunks, stride, state, cu, slot, reset, H, dk, dv};
   if (f32)
     return chunked_by_width<float, LIGHTNING>(q, k, v, nullptr, nullptr, nullptr, nullptr, nullptr, p, a, out, chunks, false, stream);
   return chunked_by_width<bf16, LIGHTNING>(q, k, v, nullptr, nullptr, nullptr, nullptr, nullptr, p, a, out, chunks, false, stream);
